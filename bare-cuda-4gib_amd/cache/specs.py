@@ -13,6 +13,8 @@ per token   ``per_token = True``.  ``page_tensors(page_tokens)`` names the tenso
             by its ``window`` (0 or absent = keep everything; W = a query reads the W tokens up to and
             including its own).  ``always_kept()`` (optional) is the number of leading tokens that stay
             whatever ``first_kept`` says: the pages that hold them are never given back before the request ends.
+            ``covering(other)`` (optional) is the spec of one stream that serves layers of both specs, or None: a
+            stream that several layers read, each as far back as its own spec says, keeps what all of them need.
 per request ``per_token = False``.  ``slot_tensors()`` names the tensors of ONE request slot
             (name -> (shape, dtype name)); the manager allocates ``[max_requests, *shape]`` of each and
             zeroes a slot when a request is admitted to it.
@@ -71,7 +73,7 @@ class FixedState:
 class PagedLatent:
     """One row of ``rank + rot`` numbers per token, in pages, shared by all heads: a low-rank latent from which keys
     and values are made, followed by a rotated key part.  Rows lie ``[page, token, rank + rot]``.  ``window`` as for
-    :class:`PagedKV`."""
+    :class:`PagedKV`.  Layers with windows of their own may read one stream: it keeps what the farthest of them reads."""
     rank: int
     rot: int
     window: int = 0
@@ -85,6 +87,12 @@ class PagedLatent:
 
     def first_kept(self, length: int) -> int:
         return max(0, length - self.window + 1) if self.window > 0 else 0
+
+    def covering(self, other) -> Optional["PagedLatent"]:
+        """The spec of one stream that serves a reader of this spec and one of ``other``; None if their rows differ."""
+        if not isinstance(other, PagedLatent) or (other.rank, other.rot) != (self.rank, self.rot):
+            return None
+        return PagedLatent(self.rank, self.rot, 0 if 0 in (self.window, other.window) else max(self.window, other.window))
 
 
 @dataclasses.dataclass(frozen=True)

@@ -8,3 +8,4 @@ from .mamenex import MamenexConfig  # noqa: F401
 from .nagezen import NagezenConfig  # noqa: F401
 from .milenex import MilenexConfig  # noqa: F401
 from .lagusun import LagusunConfig  # noqa: F401
+from .baselix import BaselixConfig  # noqa: F401

@@ -21,6 +21,10 @@ int bc4g_embed_gather(const void* table, int table_dtype, const int32_t* ids, fl
 // x[t, :] (+)= float(table[ids[t], :]) * factor  (add 0: stored, 1: added to what x holds)
 int bc4g_embed_rows(const void* table, int table_dtype, const int32_t* ids, float* out, int n_tokens, int hidden, int vocab,
                     float factor, int add, void* stream);
+// x[t, :] (+)= (float(table[ids[t], :]) + float(places[positions[t], :])) * factor, both tables of one dtype: a learned vector
+// for every position beside the token's.  NaN where a position lies outside the n_places rows.
+int bc4g_embed_placed(const void* table, const void* places, int table_dtype, const int32_t* ids, const int32_t* positions, float* out,
+                      int n_tokens, int hidden, int vocab, int n_places, float factor, int add, void* stream);
 
 // out[r, :] = x[rows ? rows[r] : r, :] * rsqrt(mean(x^2) + eps) * w      (rmsnorm.cu:16-41)
 // x is the float residual stream; out has out_dtype; w has w_dtype.
@@ -120,7 +124,7 @@ extern "C" {
 // of a k-step holds row l % 16 of the block and k 8 * (l / 16) .. + 7 of the step, zeros past n and k.
 // epilogue: 0 store bfloat16 [m, n]; 1 store float32; 2 add into float32;
 // 3 SwiGLU: every 16 rows of w are eight gate rows and the eight up rows of the same outputs
-// (n = 2 * inter), out bfloat16 [m, inter] = silu(gate) * up.
+// (n = 2 * inter), out bfloat16 [m, inter] = silu(gate) * up; 6 store max(sum, 0)^2 as bfloat16 [m, n].
 int bc4g_gemm_skinny(const void* x, const void* w, void* out, int epilogue, int m, int n, int k, void* stream);
 }
 
@@ -157,7 +161,8 @@ int bc4g_attention_mfma(const void* qkv, int q_stride, void* out, float* part_o,
 
 extern "C" {
 // bfloat16 a [m, k] times bfloat16 w [n, k] transposed on the matrix cores, any m.
-// epilogue: 0 store bfloat16; 1 store float32; 2 add into float32; 3 SwiGLU as in bc4g_gemm_skinny.
+// epilogue: 0 store bfloat16; 1 store float32; 2 add into float32; 3 SwiGLU as in bc4g_gemm_skinny; 6 store
+// max(sum, 0)^2 as bfloat16.
 // w_packed 1: w lies in the order of the weight-streaming kernel (bc4g_gemm_skinny: [ceil(n / 16)][k / 32][64 lanes][8]),
 // so that one copy of a weight serves both kernels: the kernel with operands straight into LDS reads it (k a multiple
 // of 64, operands on 16-byte boundaries).  0: w lies by rows, [n, k], for the kernel that stages its tiles through
@@ -279,7 +284,9 @@ int bc4g_rglru_scan(const float* pre, const void* u, const void* y, int dtype, c
 // rotated part of every head's query in its last rot numbers.  Elements 2i and 2i + 1 of the first `dims` numbers of
 // a rotated part turn by position * base^(-2i / dims): angles [T, dims / 2, 2] holds every row's cosines and sines
 // (bc4g_latent_angles makes it, the angles worked out in double: once a step for all layers of one rotation).  q_row,
-// dkv_row: elements from one row to the next (q and dkv may be parts of one product's rows).
+// dkv_row: elements from one row to the next (q and dkv may be parts of one product's rows).  Without a cache (a layer
+// that reads another one's latents) only the queries are rotated and dkv, g and slot_map may be null; with rot 0 only
+// the cache row is written and q and q_lat may be null.
 int bc4g_latent_angles(const int32_t* positions, float* table, int n_rows, int dims, float base, void* stream);
 int bc4g_latent_prepare(const void* q, const void* dkv, int dtype, const float* g, float eps, const float* angles,
                         const int32_t* slot_map, void* cache, float* q_lat, int n_rows, int heads, int plain, int rot,
@@ -396,6 +403,10 @@ int bc4g_embed_add(const void* table, int table_dtype, const int32_t* ids, float
 
 // z -> z Phi(z) (the exact gelu, by erf), element by element; out may be the input.
 int bc4g_gelu(const void* in, void* out, int dtype, long total, void* stream);
+// z -> max(z, 0)^2, element by element; out may be the input.
+int bc4g_squared_relu(const void* in, void* out, int dtype, long total, void* stream);
+// z = cap tanh(z / cap) in place, float32.
+int bc4g_softcap(float* z, float cap, long total, void* stream);
 
 // The choice of experts for every row (moe.hip).  logits float32 [T, >= experts] (rows logits_row apart): s =
 // softmax over the experts; choice = s + correction (null: s); the experts lie in `groups` equal groups of neighbours, a
@@ -403,8 +414,9 @@ int bc4g_gelu(const void* in, void* out, int dtype, long total, void* stream);
 // choices win (the lower index among equals).  weights float32 [T, experts]: s of the chosen, 0 elsewhere.
 // chosen int32 [T, top] (may be null).  experts at most 1024.  squash 1: s = sigmoid(logit), every expert by itself,
 // instead of the softmax.  normalize 1: the chosen experts' weights are their s divided by the sum of the chosen s
-// (+ 1e-20).  The weights are multiplied by `factor` last.
-int bc4g_moe_route(const float* logits, long logits_row, const float* correction, float* weights, int32_t* chosen,
+// (+ 1e-20).  The weights are multiplied by `factor` last.  bias float32 [experts] (may be null) is added to the logits
+// first.  squash 2: s = the logit itself, and the weights are the softmax over the chosen experts' s alone, times `factor`.
+int bc4g_moe_route(const float* logits, long logits_row, const float* bias, const float* correction, float* weights, int32_t* chosen,
                    int n_rows, int experts, int groups, int keep, int top, int squash, int normalize, float factor,
                    void* stream);
 // Plain units of all experts side by side, weighted: z [T, experts * ff + shared_ff] holds every expert's ff units and
@@ -414,7 +426,7 @@ int bc4g_routed_gelu(const void* z, void* out, int dtype, const float* weights, 
 // Clamped gated units of all experts side by side, weighted: gu [T, experts * 2 ff + 2 shared_ff] holds per expert its
 // ff gates, then its ff ups, and last the shared unit's gates and ups; out [T, experts * ff + shared_ff] =
 // weights[t, e] * g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), the shared unit
-// (its own limit) weighted by sigmoid(shared_logit[t]) (float32, rows shared_row apart; null with shared_ff 0).
+// (its own limit) weighted by sigmoid(shared_logit[t]) (float32, rows shared_row apart; null: the shared unit is added as it is).
 int bc4g_routed_glu(const void* gu, void* out, int dtype, const float* weights, const float* shared_logit, long shared_row,
                     float limit, float shared_limit, float slope, int n_rows, int experts, int ff, int shared_ff, void* stream);
 }

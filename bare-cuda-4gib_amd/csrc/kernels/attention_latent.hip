@@ -52,13 +52,13 @@ template <typename T>
 __global__ __launch_bounds__(kPrepBlock) void latent_prepare_kernel(
     const T* __restrict__ q, const T* __restrict__ dkv, const float* __restrict__ g, float eps,
     const float* __restrict__ angles, const int32_t* __restrict__ slot_map, T* __restrict__ cache,
-    float* __restrict__ q_lat, int heads, int plain, int rot, int rank, int dims, long q_row, long dkv_row) {
+    float* __restrict__ q_lat, int heads, int plain, int rot, int rank, int dims, long q_row, long dkv_row, int first_part) {
   __shared__ float scratch[16];
   extern __shared__ float cs[];                     // [dims / 2][2]: the row's cosines and sines
   const long row = blockIdx.x;
   for (int i = threadIdx.x; i < dims; i += kPrepBlock) cs[i] = angles[row * dims + i];
-  // (two workgroups a row: one norms and stores the cache row, the other rotates the queries)
-  if (blockIdx.y == 1) {
+  // (two workgroups a row, as far as there is work for them: part 0 norms and stores the cache row, part 1 rotates the queries)
+  if (static_cast<int>(blockIdx.y) + first_part == 1) {
     __syncthreads();
     const T* qr = q + row * q_row;
     float* ql = q_lat + row * heads * (rank + rot);
@@ -325,19 +325,22 @@ extern "C" int bc4g_latent_prepare(const void* q, const void* dkv, int dtype, co
                "plain=%d rot=%d rank=%d", n_rows, heads, plain, rot, rank);
   BC4G_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= rot && dims <= 8192,
                "latent_prepare: %d rotated dimensions of %d (even, at most the rotated part)", dims, rot);
-  BC4G_REQUIRE(q && dkv && g && (angles || dims == 0) && q_lat && (!cache || slot_map), "latent_prepare: a tensor is missing");
-  BC4G_REQUIRE(q_row >= static_cast<long>(heads) * (plain + rot) && dkv_row >= rank + rot, "latent_prepare: rows shorter than their parts");
-  if (n_rows == 0) return 0;
+  BC4G_REQUIRE((rot == 0 || (q && q_lat)) && (angles || dims == 0) && (!cache || (dkv && g && slot_map)),
+               "latent_prepare: a tensor is missing");
+  BC4G_REQUIRE((rot == 0 || q_row >= static_cast<long>(heads) * (plain + rot)) && (!cache || dkv_row >= rank + rot),
+               "latent_prepare: rows shorter than their parts");
+  const int first = cache ? 0 : 1, parts = (cache ? 1 : 0) + (rot > 0 ? 1 : 0);
+  if (n_rows == 0 || parts == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const size_t lds = static_cast<size_t>(dims > 0 ? dims : 2) * sizeof(float);
   if (dtype == kF32)
-    latent_prepare_kernel<float><<<dim3(n_rows, 2), kPrepBlock, lds, s>>>(static_cast<const float*>(q), static_cast<const float*>(dkv), g,
+    latent_prepare_kernel<float><<<dim3(n_rows, parts), kPrepBlock, lds, s>>>(static_cast<const float*>(q), static_cast<const float*>(dkv), g,
                                                                  eps, angles, slot_map, static_cast<float*>(cache), q_lat,
-                                                                 heads, plain, rot, rank, dims, q_row, dkv_row);
+                                                                 heads, plain, rot, rank, dims, q_row, dkv_row, first);
   else if (dtype == kBF16)
-    latent_prepare_kernel<bf16_t><<<dim3(n_rows, 2), kPrepBlock, lds, s>>>(static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(dkv),
+    latent_prepare_kernel<bf16_t><<<dim3(n_rows, parts), kPrepBlock, lds, s>>>(static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(dkv),
                                                                   g, eps, angles, slot_map, static_cast<bf16_t*>(cache),
-                                                                  q_lat, heads, plain, rot, rank, dims, q_row, dkv_row);
+                                                                  q_lat, heads, plain, rot, rank, dims, q_row, dkv_row, first);
   else return fail("latent_prepare: unknown dtype %d", dtype);
   return check_launch("latent_prepare");
 }

@@ -28,6 +28,24 @@ __global__ void embed_gather_kernel(const TT* __restrict__ table, const int32_t*
   }
 }
 
+// The same with a second table of one row a position: (table[id] + places[position]) * factor.  A position the table does
+// not have gives NaN (the host refuses such a step; nothing is read outside).
+template <typename TT>
+__global__ void embed_placed_kernel(const TT* __restrict__ table, const TT* __restrict__ places, const int32_t* __restrict__ ids,
+                                    const int32_t* __restrict__ positions, float* __restrict__ out, int hidden, int n_places,
+                                    int add, float factor) {
+  const size_t row = blockIdx.x;
+  const int at = positions[row];
+  const bool there = at >= 0 && at < n_places;
+  const TT* src = table + static_cast<size_t>(ids[row]) * hidden;
+  const TT* place = places + static_cast<size_t>(there ? at : 0) * hidden;
+  float* dst = out + row * hidden;
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+    const float v = there ? (to_float(src[i]) + to_float(place[i])) * factor : NAN;
+    dst[i] = add ? dst[i] + v : v;
+  }
+}
+
 // ---- RMSNorm ---------------------------------------------------------------
 // eps is added to the mean square; sum and rsqrt in float.
 template <typename TW, typename TO>
@@ -652,6 +670,22 @@ extern "C" int bc4g_embed_rows(const void* table, int table_dtype, const int32_t
 extern "C" int bc4g_embed_add(const void* table, int table_dtype, const int32_t* ids, float* out, int n_tokens, int hidden,
                               int vocab, void* stream) {
   return embed_rows("embed_add", table, table_dtype, ids, out, n_tokens, hidden, vocab, 1, 1.0f, stream);
+}
+
+extern "C" int bc4g_embed_placed(const void* table, const void* places, int table_dtype, const int32_t* ids, const int32_t* positions,
+                                 float* out, int n_tokens, int hidden, int vocab, int n_places, float factor, int add, void* stream) {
+  BC4G_REQUIRE(n_tokens >= 0 && hidden > 0 && vocab > 0 && n_places > 0 && table && places && ids && positions && out,
+               "embed_placed: bad arguments T=%d H=%d V=%d places=%d", n_tokens, hidden, vocab, n_places);
+  if (n_tokens == 0) return 0;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (table_dtype == kF32)
+    embed_placed_kernel<float><<<n_tokens, kBlock, 0, s>>>(static_cast<const float*>(table), static_cast<const float*>(places), ids,
+                                                          positions, out, hidden, n_places, add, factor);
+  else if (table_dtype == kBF16)
+    embed_placed_kernel<bf16_t><<<n_tokens, kBlock, 0, s>>>(static_cast<const bf16_t*>(table), static_cast<const bf16_t*>(places), ids,
+                                                           positions, out, hidden, n_places, add, factor);
+  else return fail("embed_placed: unknown table dtype %d", table_dtype);
+  return check_launch("embed_placed");
 }
 
 extern "C" int bc4g_rmsnorm(const float* x, const int32_t* rows, const void* w, int w_dtype, void* out,

@@ -42,7 +42,15 @@ constexpr int kXcds = 8;
 // kSwigluScaledBf16: the same for rows of a that lack their RMSNorm's common factor (a = bfloat16(residual * g), as the
 // product that last added to the residual left it, with every row's sum of squares in parts): a row's sums are
 // multiplied by 1 / sqrt(sum of squares / k + eps) before the activation (operands straight into LDS only).
-enum Epilogue : int { kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSwigluScaledBf16 = 5 };
+// kSquaredReluBf16: out = max(sum, 0)^2, stored as bfloat16.
+enum Epilogue : int {
+  kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSwigluScaledBf16 = 5, kSquaredReluBf16 = 6
+};
+
+__device__ inline float squared_relu(float v) {
+  const float z = fmaxf(v, 0.f);
+  return z * z;
+}
 
 constexpr int kPartSums = 8;  // chains a row's parts are added in: chain j takes parts j, j + 8, ... in ascending order, and the
                               // chains are added in order of j -- the order of the weight-streaming kernel, so the same factor
@@ -126,14 +134,18 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
         for (int e = 0; e < 8; ++e) dst[e] = from_float<bf16_t>(v[e]);
       }
     }
-  } else if (EPI == kStoreBf16 && n % 8 == 0) {
+  } else if ((EPI == kStoreBf16 || EPI == kSquaredReluBf16) && n % 8 == 0) {
     // (eight columns a thread, stored at once: 16-byte stores where 8-byte ones were, 108 -> 102 us for a wide product)
     for (int c = tid; c < ROWS * (COLS / 8); c += THREADS) {
       const int row = c / (COLS / 8), col = (c % (COLS / 8)) * 8;
       const long gm = m0 + row, gn = n0 + col;
       if (gm >= m || gn >= n) continue;
-      const floatx4 v0 = *reinterpret_cast<const floatx4*>(patch + row * kStride + col);
-      const floatx4 v1 = *reinterpret_cast<const floatx4*>(patch + row * kStride + col + 4);
+      floatx4 v0 = *reinterpret_cast<const floatx4*>(patch + row * kStride + col);
+      floatx4 v1 = *reinterpret_cast<const floatx4*>(patch + row * kStride + col + 4);
+      if constexpr (EPI == kSquaredReluBf16) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v0[e] = squared_relu(v0[e]), v1[e] = squared_relu(v1[e]);
+      }
       uint4 pk;
       pk.x = static_cast<uint32_t>(bf16_bits_from_float(v0[0])) | (static_cast<uint32_t>(bf16_bits_from_float(v0[1])) << 16);
       pk.y = static_cast<uint32_t>(bf16_bits_from_float(v0[2])) | (static_cast<uint32_t>(bf16_bits_from_float(v0[3])) << 16);
@@ -147,10 +159,14 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
       const int row = c / (COLS / 4), col = (c % (COLS / 4)) * 4;
       const long gm = m0 + row, gn = n0 + col;
       if (gm >= m || gn >= n) continue;
-      const floatx4 v = *reinterpret_cast<const floatx4*>(patch + row * kStride + col);
+      floatx4 v = *reinterpret_cast<const floatx4*>(patch + row * kStride + col);
+      if constexpr (EPI == kSquaredReluBf16) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = squared_relu(v[e]);
+      }
       const long o = gm * n + gn;
       if (vec) {
-        if constexpr (EPI == kStoreBf16) {
+        if constexpr (EPI == kStoreBf16 || EPI == kSquaredReluBf16) {
           uint2 pk;
           pk.x = static_cast<uint32_t>(bf16_bits_from_float(v[0])) | (static_cast<uint32_t>(bf16_bits_from_float(v[1])) << 16);
           pk.y = static_cast<uint32_t>(bf16_bits_from_float(v[2])) | (static_cast<uint32_t>(bf16_bits_from_float(v[3])) << 16);
@@ -166,7 +182,7 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           if (gn + e >= n) break;
-          if constexpr (EPI == kStoreBf16) static_cast<bf16_t*>(out)[o + e] = from_float<bf16_t>(v[e]);
+          if constexpr (EPI == kStoreBf16 || EPI == kSquaredReluBf16) static_cast<bf16_t*>(out)[o + e] = from_float<bf16_t>(v[e]);
           else if constexpr (EPI == kStoreF32) static_cast<float*>(out)[o + e] = v[e];
           else static_cast<float*>(out)[o + e] += v[e];
         }
@@ -789,6 +805,7 @@ extern "C" int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* 
     case kStoreBf16: e = launch_tiled<kStoreBf16>(ap, wp, out, m, n, k, s, w_packed); break;
     case kStoreF32: e = launch_tiled<kStoreF32>(ap, wp, out, m, n, k, s, w_packed); break;
     case kAccumF32: e = launch_tiled<kAccumF32>(ap, wp, out, m, n, k, s, w_packed); break;
+    case kSquaredReluBf16: e = launch_tiled<kSquaredReluBf16>(ap, wp, out, m, n, k, s, w_packed); break;
     case kSwigluBf16:
       BC4G_REQUIRE(n % 16 == 0, "gemm_mfma: SwiGLU needs blocks of eight gate and eight up rows, N=%d is no multiple of 16", n);
       e = launch_tiled<kSwigluBf16>(ap, wp, out, m, n, k, s, w_packed);

@@ -51,7 +51,7 @@ constexpr int kThreads = kWaves * kWave;
 constexpr int kRedPad = 17;
 constexpr int kStagePad = 8;     // bf16 elements appended to each staged row of x
 
-enum Epilogue : int { kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4 };
+enum Epilogue : int { kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSquaredReluBf16 = 6 };
 
 struct RopeKvArgs {
   const int32_t* positions;   // [m]
@@ -101,7 +101,7 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
     const long row0 = static_cast<long>(blockIdx.y) * args.rows_per_block;
     a.m = min(args.rows_per_block, args.m - static_cast<int>(row0));
     a.x = static_cast<const bf16_t*>(args.x) + row0 * args.k;
-    if constexpr (EPI == kStoreBf16) a.out = static_cast<bf16_t*>(args.out) + row0 * args.n;
+    if constexpr (EPI == kStoreBf16 || EPI == kSquaredReluBf16) a.out = static_cast<bf16_t*>(args.out) + row0 * args.n;
     else if constexpr (EPI == kSwigluBf16) a.out = static_cast<bf16_t*>(args.out) + row0 * (args.n / 2);
     else if constexpr (EPI == kRopeKvBf16) {
       a.out = static_cast<bf16_t*>(args.out) + row0 * args.rope.n_heads * args.rope.head_dim;
@@ -472,6 +472,9 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
     }
     if constexpr (EPI == kStoreBf16) {
       static_cast<bf16_t*>(a.out)[static_cast<long>(row) * a.n + gn] = from_float<bf16_t>(sum);
+    } else if constexpr (EPI == kSquaredReluBf16) {
+      const float z = fmaxf(sum, 0.f);
+      static_cast<bf16_t*>(a.out)[static_cast<long>(row) * a.n + gn] = from_float<bf16_t>(z * z);
     } else if constexpr (EPI == kStoreF32) {
       static_cast<float*>(a.out)[static_cast<long>(row) * a.n + gn] = sum;
     } else if constexpr (EPI == kAccumF32) {
@@ -592,6 +595,7 @@ int launch_epilogue(SkinnyArgs& a, int epilogue, hipStream_t s) {
   switch (epilogue) {
     case kStoreBf16: return launch<kStoreBf16, XMODE>(a, s);
     case kStoreF32: return launch<kStoreF32, XMODE>(a, s);
+    case kSquaredReluBf16: return launch<kSquaredReluBf16, XMODE>(a, s);
     case kAccumF32:
       if constexpr (XMODE == kPlain) return launch<kAccumF32, XMODE>(a, s);
       else return fail("gemm_skinny: adding into the stream that is being normed is not supported");

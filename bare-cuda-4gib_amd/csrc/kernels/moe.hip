@@ -7,10 +7,12 @@
 //               it is, zero elsewhere -- and the chosen experts' indices.
 //               With `squash` s = sigmoid(logit), every expert by itself; with `normalize` the chosen experts' weights are
 //               their s divided by the sum of the chosen s (+ 1e-20); the weights are multiplied by a factor last.
+//               A bias may be added to the logits first.  With squash 2 s is the logit itself, and the weights are the softmax
+//               over the chosen logits alone (times the factor).
 //   routed_gelu every expert's plain unit (the exact gelu) on its part of one wide product's row, times the row's weight for
 //               that expert; a shared unit at the end counts as it is.
 //   routed_glu  every expert's clamped gated unit on its part of one wide product's row, times the row's weight for that
-//               expert (zero for the experts the row did not choose), and a shared unit with a gate per row at the end:
+//               expert (zero for the experts the row did not choose), and a shared unit, with a gate per row or as it is, at the end:
 //               what one product over all experts' down matrices then adds up is the weighted sum of the chosen experts.
 #include <float.h>
 #include <math.h>
@@ -26,24 +28,27 @@ constexpr int kBlock = 256;
 
 // One wave a row.
 __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restrict__ logits, long logits_row,
-                                                          const float* __restrict__ correction, float* __restrict__ weights,
-                                                          int32_t* __restrict__ chosen, int experts, int groups, int keep, int top,
-                                                          int squash, int normalize, float factor) {
+                                                          const float* __restrict__ bias, const float* __restrict__ correction,
+                                                          float* __restrict__ weights, int32_t* __restrict__ chosen, int experts,
+                                                          int groups, int keep, int top, int squash, int normalize, float factor) {
   __shared__ float s_s[kMaxExperts];        // the scores
   __shared__ float c_s[kMaxExperts];        // the choices (minus infinity once taken, or outside the kept groups)
-  __shared__ float g_s[kMaxExperts];        // the groups' largest choices
+  __shared__ float g_s[kMaxExperts];        // the groups' largest choices; then (squash 2) which experts are chosen
   const int row = blockIdx.x, lane = threadIdx.x;
   const float* z = logits + row * logits_row;
+  auto logit = [&](int e) { return bias ? z[e] + bias[e] : z[e]; };
   float sum = 1.0f;
-  if (squash) {
-    for (int e = lane; e < experts; e += kWave) s_s[e] = 1.0f / (1.0f + expf(-z[e]));
+  if (squash == 2) {
+    for (int e = lane; e < experts; e += kWave) s_s[e] = logit(e);
+  } else if (squash) {
+    for (int e = lane; e < experts; e += kWave) s_s[e] = 1.0f / (1.0f + expf(-logit(e)));
   } else {
     float top_z = -INFINITY;
-    for (int e = lane; e < experts; e += kWave) top_z = fmaxf(top_z, z[e]);
+    for (int e = lane; e < experts; e += kWave) top_z = fmaxf(top_z, logit(e));
     top_z = wave_max(top_z);
     sum = 0.f;
     for (int e = lane; e < experts; e += kWave) {
-      const float p = expf(z[e] - top_z);
+      const float p = expf(logit(e) - top_z);
       s_s[e] = p;
       sum += p;
     }
@@ -54,7 +59,7 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
     const float s = s_s[e] / sum;
     s_s[e] = s;
     c_s[e] = correction ? s + correction[e] : s;
-    weights[static_cast<long>(row) * experts + e] = 0.f;
+    if (squash != 2) weights[static_cast<long>(row) * experts + e] = 0.f;
   }
   __syncthreads();
   for (int g = lane; g < groups; g += kWave) {
@@ -72,6 +77,11 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
       for (int i = 0; i < per; ++i) c_s[g * per + i] = -INFINITY;
   }
   __syncthreads();
+  if (squash == 2) {                                           // (the groups have been read: the array marks the chosen)
+    for (int e = lane; e < experts; e += kWave) g_s[e] = 0.f;
+    __syncthreads();
+  }
+  float largest = -INFINITY;                                   // of the chosen experts' scores
   float picked = 0.f;                                          // the chosen experts' scores, added up in the order of choice
   for (int n = 0; n < top; ++n) {
     float best = -INFINITY;
@@ -86,12 +96,25 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
     }
     if (at >= experts) break;                                 // fewer experts left than asked for
     picked += s_s[at];
+    largest = fmaxf(largest, s_s[at]);
     if (lane == 0) {
-      weights[static_cast<long>(row) * experts + at] = s_s[at] * (normalize ? 1.0f : factor);
+      if (squash == 2) g_s[at] = 1.0f;
+      else weights[static_cast<long>(row) * experts + at] = s_s[at] * (normalize ? 1.0f : factor);
       if (chosen) chosen[static_cast<long>(row) * top + n] = at;
       c_s[at] = -INFINITY;
     }
     __syncthreads();
+  }
+  if (squash == 2) {
+    float all = 0.f;
+    for (int e = lane; e < experts; e += kWave) {
+      const float p = g_s[e] != 0.f ? expf(s_s[e] - largest) : 0.f;
+      s_s[e] = p;
+      all += p;
+    }
+    all = wave_sum(all);
+    for (int e = lane; e < experts; e += kWave) weights[static_cast<long>(row) * experts + e] = s_s[e] / all * factor;
+    return;
   }
   if (normalize) {                                            // (the row's weights are this wave's own writes)
     const float by = factor / (picked + 1e-20f);
@@ -126,14 +149,15 @@ __global__ void routed_gelu_kernel(const T* z, T* out, const float* __restrict__
   }
 }
 
-template <typename T>
+// PIECE outputs a thread (16 bytes), all of one expert: ff and shared_ff are multiples of PIECE (1: any sizes).
+template <typename T, int PIECE>
 __global__ void routed_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, const float* __restrict__ weights,
                                   const float* __restrict__ shared_logit, long shared_row, float limit, float shared_limit,
                                   float slope, long total, int experts, int ff, int shared_ff) {
   const int out_row = experts * ff + shared_ff;
   const long in_row = 2L * out_row;
-  const long stride = static_cast<long>(blockDim.x) * gridDim.x;
-  for (long i = blockIdx.x * static_cast<long>(blockDim.x) + threadIdx.x; i < total; i += stride) {
+  const long stride = static_cast<long>(blockDim.x) * gridDim.x * PIECE;
+  for (long i = (blockIdx.x * static_cast<long>(blockDim.x) + threadIdx.x) * PIECE; i < total; i += stride) {
     const long r = i / out_row;
     const int c = static_cast<int>(i - r * out_row);
     float w, lim;
@@ -145,17 +169,32 @@ __global__ void routed_glu_kernel(const T* __restrict__ gu, T* __restrict__ out,
       g_at = r * in_row + 2L * e * ff + (c - e * ff);
       width = ff, lim = limit;
     } else {
-      w = 1.0f / (1.0f + expf(-shared_logit[r * shared_row]));
+      w = shared_logit ? 1.0f / (1.0f + expf(-shared_logit[r * shared_row])) : 1.0f;
       g_at = r * in_row + 2L * experts * ff + (c - experts * ff);
       width = shared_ff, lim = shared_limit;
     }
-    float y = 0.f;
+    __align__(16) T gates[PIECE];
+    __align__(16) T ups[PIECE];
     if (w != 0.f) {
-      const float g = fminf(to_float(gu[g_at]), lim);
-      const float u = fminf(fmaxf(to_float(gu[g_at + width]), -lim), lim);
-      y = w * (g / (1.0f + expf(-slope * g)) * (u + 1.0f));
+      if (PIECE == 1) {
+        gates[0] = gu[g_at], ups[0] = gu[g_at + width];
+      } else {
+        *reinterpret_cast<uint4*>(gates) = *reinterpret_cast<const uint4*>(gu + g_at);
+        *reinterpret_cast<uint4*>(ups) = *reinterpret_cast<const uint4*>(gu + g_at + width);
+      }
     }
-    out[i] = from_float<T>(y);
+#pragma unroll
+    for (int e = 0; e < PIECE; ++e) {
+      float y = 0.f;
+      if (w != 0.f) {
+        const float g = fminf(to_float(gates[e]), lim);
+        const float u = fminf(fmaxf(to_float(ups[e]), -lim), lim);
+        y = w * (g / (1.0f + expf(-slope * g)) * (u + 1.0f));
+      }
+      gates[e] = from_float<T>(y);
+    }
+    if (PIECE == 1) out[i] = gates[0];
+    else *reinterpret_cast<uint4*>(out + i) = *reinterpret_cast<const uint4*>(gates);
   }
 }
 
@@ -164,15 +203,16 @@ __global__ void routed_glu_kernel(const T* __restrict__ gu, T* __restrict__ out,
 
 using namespace bc4g;
 
-extern "C" int bc4g_moe_route(const float* logits, long logits_row, const float* correction, float* weights, int32_t* chosen,
-                              int n_rows, int experts, int groups, int keep, int top, int squash, int normalize, float factor,
+extern "C" int bc4g_moe_route(const float* logits, long logits_row, const float* bias, const float* correction, float* weights,
+                              int32_t* chosen, int n_rows, int experts, int groups, int keep, int top, int squash, int normalize, float factor,
                               void* stream) {
   BC4G_REQUIRE(n_rows >= 0 && experts > 0 && experts <= kMaxExperts && logits && weights && logits_row >= experts,
                "moe_route: bad arguments rows=%d experts=%d (at most %d)", n_rows, experts, kMaxExperts);
   BC4G_REQUIRE(groups > 0 && experts % groups == 0 && keep > 0 && keep <= groups && top > 0 && top <= experts,
                "moe_route: %d experts in %d groups of which %d are kept, %d chosen", experts, groups, keep, top);
+  BC4G_REQUIRE(squash >= 0 && squash <= 2, "moe_route: squash %d (0 softmax, 1 sigmoid, 2 the logits)", squash);
   if (n_rows == 0) return 0;
-  moe_route_kernel<<<n_rows, kWave, 0, static_cast<hipStream_t>(stream)>>>(logits, logits_row, correction, weights, chosen,
+  moe_route_kernel<<<n_rows, kWave, 0, static_cast<hipStream_t>(stream)>>>(logits, logits_row, bias, correction, weights, chosen,
                                                                            experts, groups, keep, top, squash, normalize,
                                                                            factor);
   return check_launch("moe_route");
@@ -210,20 +250,26 @@ extern "C" int bc4g_routed_glu(const void* gu, void* out, int dtype, const float
                                int shared_ff, void* stream) {
   BC4G_REQUIRE(n_rows >= 0 && experts >= 0 && ff >= 0 && shared_ff >= 0 && experts * ff + shared_ff > 0 && gu && out && gu != out,
                "routed_glu: bad arguments rows=%d experts=%d ff=%d shared=%d", n_rows, experts, ff, shared_ff);
-  BC4G_REQUIRE((experts == 0 || weights) && (shared_ff == 0 || shared_logit), "routed_glu: the weights or the shared gate are missing");
+  BC4G_REQUIRE(experts == 0 || weights, "routed_glu: the weights are missing");
   const long total = static_cast<long>(n_rows) * (static_cast<long>(experts) * ff + shared_ff);
   if (total == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const long blocks = (total + kBlock - 1) / kBlock;
+  const int piece = dtype == kF32 ? 4 : 8;      // elements in 16 bytes
+  const bool pieces = ff % piece == 0 && shared_ff % piece == 0 && reinterpret_cast<uintptr_t>(gu) % 16 == 0 &&
+                      reinterpret_cast<uintptr_t>(out) % 16 == 0;
+  const long threads = pieces ? total / piece : total;
+  const long blocks = (threads + kBlock - 1) / kBlock;
   const int grid = static_cast<int>(blocks > 65535 ? 65535 : blocks);
-  if (dtype == kF32)
-    routed_glu_kernel<float><<<grid, kBlock, 0, s>>>(static_cast<const float*>(gu), static_cast<float*>(out), weights, shared_logit,
-                                                     shared_row, limit, shared_limit, slope, total, experts, ff, shared_ff);
-  else if (dtype == kBF16)
-    routed_glu_kernel<bf16_t><<<grid, kBlock, 0, s>>>(static_cast<const bf16_t*>(gu), static_cast<bf16_t*>(out), weights,
-                                                      shared_logit, shared_row, limit, shared_limit, slope, total, experts, ff,
-                                                      shared_ff);
-  else
+#define BC4G_ROUTED_GLU(T, P)                                                                                              \
+  routed_glu_kernel<T, P><<<grid, kBlock, 0, s>>>(static_cast<const T*>(gu), static_cast<T*>(out), weights, shared_logit, shared_row, \
+                                                  limit, shared_limit, slope, total, experts, ff, shared_ff)
+  if (dtype == kF32) {
+    if (pieces) BC4G_ROUTED_GLU(float, 4); else BC4G_ROUTED_GLU(float, 1);
+  } else if (dtype == kBF16) {
+    if (pieces) BC4G_ROUTED_GLU(bf16_t, 8); else BC4G_ROUTED_GLU(bf16_t, 1);
+  } else {
     return fail("routed_glu: unknown dtype %d", dtype);
+  }
+#undef BC4G_ROUTED_GLU
   return check_launch("routed_glu");
 }

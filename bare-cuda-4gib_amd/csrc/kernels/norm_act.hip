@@ -109,6 +109,40 @@ __global__ void gelu_kernel(const T* __restrict__ in, T* __restrict__ out, long 
   }
 }
 
+// max(z, 0)^2, element by element; PIECE elements a thread (16 bytes; 1: any count).
+template <typename T, int PIECE>
+__global__ void squared_relu_kernel(const T* in, T* out, long total) {      // (out may be in)
+  const long stride = static_cast<long>(blockDim.x) * gridDim.x * PIECE;
+  for (long i = (blockIdx.x * static_cast<long>(blockDim.x) + threadIdx.x) * PIECE; i < total; i += stride) {
+    __align__(16) T piece[PIECE];
+    if (PIECE == 1) piece[0] = in[i];
+    else *reinterpret_cast<uint4*>(piece) = *reinterpret_cast<const uint4*>(in + i);
+#pragma unroll
+    for (int e = 0; e < PIECE; ++e) {
+      const float z = fmaxf(to_float(piece[e]), 0.f);
+      piece[e] = from_float<T>(z * z);
+    }
+    if (PIECE == 1) out[i] = piece[0];
+    else *reinterpret_cast<uint4*>(out + i) = *reinterpret_cast<const uint4*>(piece);
+  }
+}
+
+// z = cap tanh(z / cap) in place, four elements a thread (V 1: any count).
+template <int V>
+__global__ void softcap_kernel(float* __restrict__ z, float cap, long total) {
+  const float inv = 1.0f / cap;
+  const long stride = static_cast<long>(blockDim.x) * gridDim.x * V;
+  for (long i = (blockIdx.x * static_cast<long>(blockDim.x) + threadIdx.x) * V; i < total; i += stride) {
+    if (V == 4) {
+      const float4 v = *reinterpret_cast<const float4*>(z + i);
+      *reinterpret_cast<float4*>(z + i) = make_float4(cap * tanhf(v.x * inv), cap * tanhf(v.y * inv), cap * tanhf(v.z * inv),
+                                                      cap * tanhf(v.w * inv));
+    } else {
+      z[i] = cap * tanhf(z[i] * inv);
+    }
+  }
+}
+
 int grid_for(long total) {
   const long g = (total + kBlock - 1) / kBlock;
   return static_cast<int>(g < 1 ? 1 : (g > 65535 ? 65535 : g));
@@ -240,6 +274,30 @@ extern "C" int bc4g_gelu(const void* in, void* out, int dtype, long total, void*
   else if (dtype == kBF16) gelu_kernel<bf16_t><<<grid_for(total), kBlock, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), total);
   else return fail("gelu: unknown dtype %d", dtype);
   return check_launch("gelu");
+}
+
+extern "C" int bc4g_squared_relu(const void* in, void* out, int dtype, long total, void* stream) {
+  BC4G_REQUIRE(total >= 0 && in && out, "squared_relu: bad arguments (%ld elements)", total);
+  if (total == 0) return 0;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const int piece = dtype == kF32 ? 4 : 8;      // elements in 16 bytes
+  const bool pieces = total % piece == 0 && reinterpret_cast<uintptr_t>(in) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+#define BC4G_RELU2(T, P) \
+  squared_relu_kernel<T, P><<<grid_for(total / P), kBlock, 0, s>>>(static_cast<const T*>(in), static_cast<T*>(out), total)
+  if (dtype == kF32) { if (pieces) BC4G_RELU2(float, 4); else BC4G_RELU2(float, 1); }
+  else if (dtype == kBF16) { if (pieces) BC4G_RELU2(bf16_t, 8); else BC4G_RELU2(bf16_t, 1); }
+  else return fail("squared_relu: unknown dtype %d", dtype);
+#undef BC4G_RELU2
+  return check_launch("squared_relu");
+}
+
+extern "C" int bc4g_softcap(float* z, float cap, long total, void* stream) {
+  BC4G_REQUIRE(total >= 0 && z && cap > 0.f, "softcap: bad arguments (%ld elements, cap %g)", total, cap);
+  if (total == 0) return 0;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (total % 4 == 0 && reinterpret_cast<uintptr_t>(z) % 16 == 0) softcap_kernel<4><<<grid_for(total / 4), kBlock, 0, s>>>(z, cap, total);
+  else softcap_kernel<1><<<grid_for(total), kBlock, 0, s>>>(z, cap, total);
+  return check_launch("softcap");
 }
 
 extern "C" int bc4g_rmsnorm_shift(const float* x, const float* w, const float* mix, void* out, void* state, int dtype,

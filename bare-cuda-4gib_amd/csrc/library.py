@@ -18,6 +18,7 @@ _F = c_float
 _SIGNATURES = {
     "bc4g_embed_gather": [_P, _I, _P, _P, _I, _I, _I, _P],
     "bc4g_embed_rows": [_P, _I, _P, _P, _I, _I, _I, _F, _I, _P],
+    "bc4g_embed_placed": [_P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _F, _I, _P],
     "bc4g_rmsnorm": [_P, _P, _P, _I, _P, _I, _I, _I, _F, _P],
     "bc4g_rmsnorm_groups": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P],
     "bc4g_stream_update": [_P, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _I, _F, _P],
@@ -71,7 +72,9 @@ _SIGNATURES = {
                             _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P, c_long, _P],
     "bc4g_embed_add": [_P, _I, _P, _P, _I, _I, _I, _P],
     "bc4g_gelu": [_P, _P, _I, c_long, _P],
-    "bc4g_moe_route": [_P, c_long, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
+    "bc4g_squared_relu": [_P, _P, _I, c_long, _P],
+    "bc4g_softcap": [_P, _F, c_long, _P],
+    "bc4g_moe_route": [_P, c_long, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
     "bc4g_routed_gelu": [_P, _P, _I, _P, _I, _I, _I, _I, _P],
     "bc4g_routed_glu": [_P, _P, _I, _P, _P, c_long, _F, _F, _F, _I, _I, _I, _I, _P],
     "bc4g_attention_latent_mfma": [_P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],

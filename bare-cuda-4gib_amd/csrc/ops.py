@@ -121,6 +121,28 @@ def embed_add(table: torch.Tensor, ids: torch.Tensor, x: torch.Tensor, factor: f
     return x
 
 
+def embed_placed(table: torch.Tensor, places: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, factor: float = 1.0,
+                 add_to: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """(float(table[ids[t], :]) + float(places[positions[t], :])) * factor as float32 [T, H]: a learned vector for every
+    position beside the token's.  ``add_to``: added in place to that float32 stream instead.  The ids must be known to
+    lie in the vocabulary and the positions in the table (a position outside gives NaN)."""
+    _dev("embed_placed", table, places, ids, positions, add_to)
+    (vocab, hidden), n = table.shape, ids.numel()
+    _i32("embed_placed", "ids", ids, n)
+    _i32("embed_placed", "positions", positions, n)
+    if places.dtype != table.dtype or places.dim() != 2 or places.shape[1] != hidden:
+        raise KernelError(f"embed_placed: the positions' table must be {table.dtype} [positions, {hidden}], got {places.dtype} {tuple(places.shape)}")
+    out = add_to
+    if out is None:
+        out = torch.empty((n, hidden), dtype=torch.float32, device=table.device)
+    elif out.dtype != torch.float32 or tuple(out.shape) != (n, hidden):
+        raise KernelError(f"embed_placed: the stream must be float32 [{n}, {hidden}], got {out.dtype} {tuple(out.shape)}")
+    library.call("bc4g_embed_placed", _ptr(table), _ptr(places), _code(table, "embed_placed"), _ptr(ids), _ptr(positions), _ptr(out), n,
+                 hidden, vocab, places.shape[0], float(factor), 0 if add_to is None else 1, _stream(),
+                 cost=lambda: (2.0 * n * hidden, n * hidden * (2 * table.element_size() + (4 if add_to is None else 8))))
+    return out
+
+
 def embed_beside(x: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, out_dtype: torch.dtype, factor: float = 1.0) -> torch.Tensor:
     """[T, 2 H] in ``out_dtype``: row t is the float32 stream's row x[t, :] followed by table[ids[t], :] * factor -- the
     operand of a product over the stream and the embedding of the same token."""
@@ -628,6 +650,7 @@ def streams_weights(m: int, n: int, k: int) -> bool:
 
 
 EPI_STORE_BF16, EPI_STORE_F32, EPI_ACCUM_F32, EPI_SWIGLU = 0, 1, 2, 3
+EPI_SQUARED_RELU = 6      # max(sum, 0)^2 stored as bfloat16
 
 
 def _fast_operands(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -636,13 +659,14 @@ def _fast_operands(a: torch.Tensor, w: torch.Tensor) -> bool:
 
 
 def gemm_fast(a: torch.Tensor, w, out_dtype=None,
-              accumulate_into: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+              accumulate_into: Optional[torch.Tensor] = None, squared_relu: bool = False) -> Optional[torch.Tensor]:
     """The matrix-core product where a kernel takes these operands (bfloat16, k a multiple of
     8), else None (the caller then uses the plain float kernel).  Up to 64 rows the weights
     are streamed once (a decode step); a wide output goes to the tiled kernel from 24 rows on,
-    everything from 65."""
+    everything from 65.  ``squared_relu``: the result is max(product, 0)^2, applied to the float sums
+    inside the product's kernel (a bfloat16 result only)."""
     w, packed = _weight(w)
-    if not _fast_operands(a, w):
+    if not _fast_operands(a, w) or (squared_relu and (accumulate_into is not None or (out_dtype or a.dtype) != torch.bfloat16)):
         return None
     _dev("gemm", a, w, accumulate_into)
     m, k = a.shape
@@ -656,7 +680,7 @@ def gemm_fast(a: torch.Tensor, w, out_dtype=None,
         if out_dtype not in (torch.bfloat16, torch.float32):
             return None
         out = torch.empty((m, n), dtype=out_dtype, device=a.device)
-        epi = EPI_STORE_BF16 if out_dtype == torch.bfloat16 else EPI_STORE_F32
+        epi = EPI_SQUARED_RELU if squared_relu else EPI_STORE_BF16 if out_dtype == torch.bfloat16 else EPI_STORE_F32
     out_bytes = 8 if accumulate_into is not None else out.element_size()
     if streams_weights(m, n, k):
         packed = packed if packed is not None else pack_weight(_rows(w))      # (packing per call: tests only)
@@ -686,7 +710,7 @@ def gemm_normed_supported(x: torch.Tensor, n_rows: int, g: torch.Tensor, w) -> b
 def gemm_normed(x: torch.Tensor, rows: Optional[torch.Tensor], n_rows: int, g: torch.Tensor, eps: float,
                 w, epilogue: int) -> torch.Tensor:
     """rmsnorm(x[rows]) W^T with the norm fused into the product (see gemm_skinny.hip): epilogue
-    EPI_STORE_BF16, EPI_STORE_F32 or EPI_SWIGLU (w = gate rows then up rows)."""
+    EPI_STORE_BF16, EPI_STORE_F32, EPI_SQUARED_RELU or EPI_SWIGLU (w = gate rows then up rows)."""
     w, packed = _weight(w)
     packed = packed if packed is not None else pack_weight(_rows(w))
     _dev("gemm_normed", x, rows, g, w)
@@ -699,7 +723,7 @@ def gemm_normed(x: torch.Tensor, rows: Optional[torch.Tensor], n_rows: int, g: t
         raise KernelError("gemm_normed: without row indices every row of x is used")
     if epilogue == EPI_SWIGLU:
         out = torch.empty((n_rows, n // 2), dtype=torch.bfloat16, device=x.device)
-    elif epilogue == EPI_STORE_BF16:
+    elif epilogue in (EPI_STORE_BF16, EPI_SQUARED_RELU):
         out = torch.empty((n_rows, n), dtype=torch.bfloat16, device=x.device)
     elif epilogue == EPI_STORE_F32:
         out = torch.empty((n_rows, n), dtype=torch.float32, device=x.device)
@@ -849,7 +873,7 @@ def gemm_prenormed_supported(pre: Prenormed, w, epilogue: Optional[int] = None) 
 
 def gemm_prenormed(pre: Prenormed, w, epilogue: int) -> torch.Tensor:
     """rmsnorm(residual) w^T from what gemm_accumulate_emit left: epilogue EPI_STORE_BF16,
-    EPI_STORE_F32 or EPI_SWIGLU (w in blocks of eight gate and eight up rows)."""
+    EPI_STORE_F32, EPI_SQUARED_RELU or EPI_SWIGLU (w in blocks of eight gate and eight up rows)."""
     w, packed = _weight(w)
     tiled_w = _tiled_weight(w, packed)
     packed = packed if packed is not None else pack_weight(_rows(w))
@@ -858,7 +882,7 @@ def gemm_prenormed(pre: Prenormed, w, epilogue: int) -> torch.Tensor:
     n = w.shape[0]
     if epilogue == EPI_SWIGLU:
         out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=w.device)
-    elif epilogue == EPI_STORE_BF16:
+    elif epilogue in (EPI_STORE_BF16, EPI_SQUARED_RELU):
         out = torch.empty((m, n), dtype=torch.bfloat16, device=w.device)
     elif epilogue == EPI_STORE_F32:
         out = torch.empty((m, n), dtype=torch.float32, device=w.device)
@@ -1376,10 +1400,10 @@ def attention_latent_mfma_takes(cache: torch.Tensor, rank: int, rot: int) -> boo
             and cache.data_ptr() % 16 == 0)
 
 
-def latent_splits(seq_start, heads: int, max_kv_len: int) -> int:
+def latent_splits(seq_start, heads: int, max_kv_len: int, window: int = 0) -> int:
     """Into how many parts the matrix-core kernel cuts every walk over the keys: one where the step's rows fill the
     GPU by themselves (a workgroup takes four tiles of 16 (token, head) pairs of one request), else as many as bring
-    the workgroups to twice that, while a part keeps a key tile of 32."""
+    the workgroups to twice that, while a part keeps a key tile of 32 (of a ``window``'s keys, if there is one)."""
     hb = min(heads, 16)
     tpt, n_hg = 16 // hb, -(-heads // hb)
     tiles = [-(-int(seq_start[s + 1] - seq_start[s]) // tpt) * n_hg for s in range(len(seq_start) - 1)]
@@ -1387,7 +1411,10 @@ def latent_splits(seq_start, heads: int, max_kv_len: int) -> int:
     groups = sum(tiles) if max(tiles, default=0) < 4 else sum(-(-n // 4) for n in tiles)
     if groups >= LATENT_ENOUGH_GROUPS or groups == 0:
         return 1
-    key_tiles = -(-max_kv_len // 32)
+    span = max_kv_len
+    if window > 0:          # (a workgroup's tokens together see the window and its own tokens before the last)
+        span = min(span, window + 4 * tpt + 31)
+    key_tiles = -(-span // 32)
     return max(1, min(-(-2 * LATENT_ENOUGH_GROUPS // groups), key_tiles, LATENT_MAX_SPLITS))
 
 
@@ -1403,22 +1430,28 @@ def latent_angles(positions: torch.Tensor, dims: int, base: float) -> torch.Tens
     return table
 
 
-def latent_prepare(q: torch.Tensor, dkv: torch.Tensor, g: torch.Tensor, eps: float, angles: Optional[torch.Tensor],
+def latent_prepare(q: torch.Tensor, dkv: Optional[torch.Tensor], g: Optional[torch.Tensor], eps: float, angles: Optional[torch.Tensor],
                    slot_map: Optional[torch.Tensor], cache: Optional[torch.Tensor], q_lat: torch.Tensor, heads: int, plain: int,
                    rot: int, rank: int, dims: int) -> None:
     """Writes [rmsnorm(dkv[:, :rank]) * g | rotate(dkv[:, rank:])] into every row's cache slot (``cache`` None: nowhere)
     and every head's rotated query part into q_lat[:, h, rank:].  ``angles``: latent_angles of the rows (None where
-    nothing is rotated, dims 0)."""
+    nothing is rotated, dims 0).  Without a cache dkv and g may be None: only the queries are rotated."""
     _dev("latent_prepare", g, angles, slot_map, cache, q_lat)
-    q_row, dkv_row = _rows_of("latent_prepare", "q", q), _rows_of("latent_prepare", "dkv", dkv)   # (parts of one product's rows)
+    if cache is None and rot == 0:
+        return                  # nothing to write
+    q_row = _rows_of("latent_prepare", "q", q)                 # (q and dkv may be parts of one product's rows)
+    dkv_row = _rows_of("latent_prepare", "dkv", dkv) if dkv is not None else 0
     t = q.shape[0]
-    if q.dtype != dkv.dtype or tuple(q.shape) != (t, heads * (plain + rot)) or tuple(dkv.shape) != (t, rank + rot):
-        raise KernelError(f"latent_prepare: q {tuple(q.shape)} / dkv {tuple(dkv.shape)} do not fit heads={heads} plain={plain} rot={rot} rank={rank}")
+    if tuple(q.shape) != (t, heads * (plain + rot)) or (dkv is not None and (q.dtype != dkv.dtype or tuple(dkv.shape) != (t, rank + rot))):
+        raise KernelError(f"latent_prepare: q {tuple(q.shape)} / dkv {tuple(dkv.shape) if dkv is not None else None} do not fit "
+                          f"heads={heads} plain={plain} rot={rot} rank={rank}")
     _f32("latent_prepare", "g", g, (rank,))
     _f32("latent_prepare", "q_lat", q_lat, (t, heads, rank + rot))
     if dims:
         _f32("latent_prepare", "angles", angles, (t, dims // 2, 2))
     if cache is not None:
+        if dkv is None or g is None:
+            raise KernelError("latent_prepare: a cache row is made of dkv and g")
         if cache.dtype != q.dtype or cache.dim() != 3 or cache.shape[2] != rank + rot:
             raise KernelError(f"latent_prepare: the cache must be {q.dtype} [pages, page_tokens, {rank + rot}], got {cache.dtype} {tuple(cache.shape)}")
         _i32("latent_prepare", "slot_map", slot_map, t)
@@ -1464,7 +1497,7 @@ def attention_latent(q_lat: torch.Tensor, cache: torch.Tensor, sink: Optional[to
     if attention_latent_mfma_takes(cache, rank, rot):
         _i32("attention_latent", "seq_start", ctx.seq_start_dev, ctx.n_seqs + 1)
         _i32("attention_latent", "seq_ctx", ctx.seq_ctx_dev, ctx.n_seqs)
-        n_splits = latent_splits(ctx.seq_start, heads, ctx.max_kv_len)
+        n_splits = latent_splits(ctx.seq_start, heads, ctx.max_kv_len, int(window))
         most = max(int(ctx.seq_start[s + 1] - ctx.seq_start[s]) for s in range(ctx.n_seqs))
         part_o = part_ml = None
         if n_splits > 1:
@@ -1904,6 +1937,31 @@ def attention_talk(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
 
 # ---- activations and routing of a mixture of experts ------------------------------------------------------------------------
 
+def squared_relu(z: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """max(z, 0)^2, element by element; ``out`` may be z itself."""
+    _dev("squared_relu", z, out)
+    if not z.is_contiguous():
+        raise KernelError("squared_relu: the input's elements must lie side by side")
+    if out is None:
+        out = torch.empty_like(z)
+    elif out.dtype != z.dtype or out.shape != z.shape or not out.is_contiguous():
+        raise KernelError("squared_relu: out must have the input's dtype and shape")
+    total = z.numel()
+    library.call("bc4g_squared_relu", _ptr(z), _ptr(out), _code(z, "squared_relu"), total, _stream(),
+                 cost=lambda: (2.0 * total, 2 * total * z.element_size()))
+    return out
+
+
+def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """z = cap tanh(z / cap) in place on a float32 tensor."""
+    _dev("softcap", z)
+    if z.dtype != torch.float32 or not z.is_contiguous() or not cap > 0:
+        raise KernelError(f"softcap: float32 elements side by side and a positive cap, got {z.dtype} and {cap}")
+    total = z.numel()
+    library.call("bc4g_softcap", _ptr(z), float(cap), total, _stream(), cost=lambda: (10.0 * total, 8 * total))
+    return z
+
+
 def gelu(z: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """z Phi(z), the exact gelu, element by element; ``out`` may be z itself."""
     _dev("gelu", z, out)
@@ -1924,23 +1982,28 @@ MOE_MAX_EXPERTS = 1024
 
 def moe_route(logits: torch.Tensor, experts: int, top: int, groups: int = 1, keep: int = 1,
               correction: Optional[torch.Tensor] = None, want_chosen: bool = False, squash: bool = False,
-              normalize: bool = False, factor: float = 1.0):
+              normalize: bool = False, factor: float = 1.0, bias: Optional[torch.Tensor] = None, over_chosen: bool = False):
     """The choice of experts for every row: logits float32 [T, >= experts] (the first ``experts`` columns count; rows may
     be parts of wider rows).  s = softmax(logits); the choice goes by s + correction; only experts of the ``keep`` best of
     ``groups`` equal groups of neighbours (a group counts by its largest choice) can be chosen; the ``top`` largest win.
     ``squash``: s = sigmoid(logits), every expert by itself, instead of the softmax.  ``normalize``: the chosen experts'
     weights are their s divided by the sum of the chosen s (+ 1e-20).  ``factor`` multiplies the weights last.
+    ``bias`` float32 [experts] is added to the logits first.  ``over_chosen``: s is the logit itself, and the weights are the
+    softmax over the chosen logits alone (times ``factor``).
     Returns weights float32 [T, experts] -- s of the chosen, zero elsewhere -- and, if asked, the chosen int32 [T, top]."""
-    _dev("moe_route", correction)
+    _dev("moe_route", correction, bias)
+    if over_chosen and (squash or normalize):
+        raise KernelError("moe_route: a softmax over the chosen logits takes neither squash nor normalize")
     row = _part_of_rows("moe_route", "logits", logits, experts)
     if logits.dtype != torch.float32:
         raise KernelError(f"moe_route: logits must be float32, got {logits.dtype}")
     _f32("moe_route", "correction", correction, (experts,))
+    _f32("moe_route", "bias", bias, (experts,))
     t = logits.shape[0]
     weights = torch.empty((t, experts), dtype=torch.float32, device=logits.device)
     chosen = torch.empty((t, top), dtype=torch.int32, device=logits.device) if want_chosen else None
-    library.call("bc4g_moe_route", _ptr(logits), row, _ptr(correction), _ptr(weights), _ptr(chosen), t, experts, groups, keep, top,
-                 1 if squash else 0, 1 if normalize else 0, float(factor), _stream(),
+    library.call("bc4g_moe_route", _ptr(logits), row, _ptr(bias), _ptr(correction), _ptr(weights), _ptr(chosen), t, experts, groups, keep, top,
+                 2 if over_chosen else 1 if squash else 0, 1 if normalize else 0, float(factor), _stream(),
                  cost=lambda: (8.0 * t * experts * (1 + top), 8.0 * t * experts))
     return (weights, chosen) if want_chosen else weights
 
@@ -1970,7 +2033,7 @@ def routed_glu(gu: torch.Tensor, weights: Optional[torch.Tensor], experts: int, 
     """gu [T, experts * 2 ff + 2 shared_ff]: per expert its ff gates, then its ff ups, and last the shared unit's.  Returns
     [T, experts * ff + shared_ff]: weights[t, e] * g sigmoid(slope g) (u + 1) with g = min(gate, limit),
     u = clamp(up, -limit, limit); the shared unit (its own limit) times sigmoid(shared_logit[t]) (float32 [T, 1], may be a
-    part of wider rows)."""
+    part of wider rows), or as it is without a shared_logit."""
     _dev("routed_glu", gu, weights)
     t = gu.shape[0]
     if gu.dim() != 2 or gu.shape[1] != 2 * (experts * ff + shared_ff) or not gu.is_contiguous():
@@ -1978,9 +2041,9 @@ def routed_glu(gu: torch.Tensor, weights: Optional[torch.Tensor], experts: int, 
     if experts:
         _f32("routed_glu", "weights", weights, (t, experts))
     shared_row = 0
-    if shared_ff:
-        if shared_logit is None or shared_logit.dtype != torch.float32 or shared_logit.shape[0] != t:
-            raise KernelError("routed_glu: the shared unit needs a float32 gate logit for every row")
+    if shared_ff and shared_logit is not None:
+        if shared_logit.dtype != torch.float32 or shared_logit.shape[0] != t:
+            raise KernelError("routed_glu: the shared unit's gate is a float32 logit for every row")
         shared_row = _part_of_rows("routed_glu", "shared_logit", shared_logit, 1)
     out = torch.empty((t, experts * ff + shared_ff), dtype=gu.dtype, device=gu.device)
     library.call("bc4g_routed_glu", _ptr(gu), _ptr(out), _code(gu, "routed_glu"), _ptr(weights), _ptr(shared_logit), shared_row,

@@ -69,10 +69,13 @@ class Executor:
         if model.rt is None:
             raise EngineError("executor: the model has no weights bound")
         # (reference: Model::load, engine/src/model.cpp:429-433.  ``beyond_positions``: a program that replays given
-        # ids and serves nobody may say that it wants positions the configuration does not promise -- nothing here
-        # keeps a table of them -- and takes the answers for what they are.)
+        # ids and serves nobody may say that it wants positions the configuration does not promise, and takes the
+        # answers for what they are.)
         if max_tokens > model.max_seq_len and not beyond_positions:
             raise EngineError(f"executor: max_tokens {max_tokens} is beyond the model's {model.max_seq_len} positions")
+        # A part that looks positions up in a table has none beyond it, whatever the caller says: there a request ends.
+        limits = [p.position_limit for p in model.all_parts() if getattr(p, "position_limit", 0)]
+        max_tokens = min([max_tokens, *limits])
         self.model = model
         self.rt = model.rt
         self.max_batch_tokens = max_batch_tokens

@@ -136,7 +136,8 @@ class Model:
     def cache_streams(self) -> Dict[Hashable, object]:
         """Cache stream id -> spec, from the schedule: the entry that writes a
         stream decides its spec; an entry may only read a stream that some
-        entry writes."""
+        entry writes.  A reader whose spec differs must be one the writer's can
+        be widened to cover (``covering``: the same rows, kept longer)."""
         streams: Dict[Hashable, object] = {}
         for e in self.schedule:
             if e.cache is None or not e.writes:
@@ -152,9 +153,12 @@ class Model:
             if e.cache not in streams:
                 raise ConfigError(f"schedule entry for layer {e.layer} reads cache stream {e.cache!r}, "
                                   "which no entry writes")
-            mixer = self.layers[e.layer].mixer
-            if self._cache_spec(e.layer) != streams[e.cache]:
-                raise ConfigError(f"layer {e.layer} uses cache stream {e.cache!r} with another spec than its writer")
+            mixer, spec = self.layers[e.layer].mixer, self._cache_spec(e.layer)
+            if spec != streams[e.cache]:
+                both = streams[e.cache].covering(spec) if hasattr(streams[e.cache], "covering") else None
+                if both is None:
+                    raise ConfigError(f"layer {e.layer} uses cache stream {e.cache!r} with another spec than its writer")
+                streams[e.cache] = both
             layout = mixer.cache_layout() if hasattr(mixer, "cache_layout") else None
             if layouts.setdefault(e.cache, layout) != layout:
                 raise ConfigError(f"layers sharing cache stream {e.cache!r} keep a head's dimensions in "

@@ -9,7 +9,7 @@ from ..csrc import ops
 from ..errors import ConfigError
 from ..weights.loader import WeightSpec
 from .base import Part, register_part
-from .linear import linear, linear_swiglu
+from .linear import linear, linear_squared_relu, linear_swiglu
 
 
 class SwiGLU(Part):
@@ -141,6 +141,42 @@ class DenseGELU(Part):
         linear(ops.gelu(z, out=z), self.w_down, accumulate_into=residual, ctx=ctx)
 
 
+class DenseSquaredReLU(Part):
+    """x += Wd max(Wu h, 0)^2, no biases; the activation is applied to the first product's float sums."""
+    category = "feedforward"
+    graph_safe = True     # launches kernels only: may run inside a captured graph
+    accepts_lazy_norm = True
+    adds_one_product = True   # the output is one last product through linear(): a block may hand it ops.Fresh
+
+    def __init__(self, hidden_size: int, intermediate_size: int):
+        self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+        if self.intermediate_size <= 0:
+            raise ConfigError(f"dense feed-forward: size {intermediate_size} must be positive")
+        self.w_up = self.w_down = None
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        h, i = self.hidden_size, self.intermediate_size
+        return {"up": WeightSpec((i, h)), "down": WeightSpec((h, i))}
+
+    def bind(self, tensors, rt) -> None:
+        self.w_up = ops.StreamedWeight(tensors["up"])
+        self.w_down = ops.StreamedWeight(tensors["down"])
+        self.act_dtype = rt.act_dtype
+
+    def step_work(self, batch, rows: int, elem: int):
+        flops, nbytes = super().step_work(batch, rows, elem)
+        return flops + 2.0 * rows * self.intermediate_size, nbytes
+
+    def wants_prepared_norm(self, n_rows: int) -> bool:
+        """Whether the first product, at this many rows, is better served by a norm that the product before prepared
+        than by fusing the norm or running it: the weight's own plan says (ops.LinearPlan.wants_prepared)."""
+        return self.act_dtype == torch.bfloat16 and self.w_up.plan.wants_prepared(n_rows)
+
+    def forward(self, h, ctx, residual) -> None:
+        act = linear_squared_relu(h, self.w_up, self.act_dtype)
+        linear(act, self.w_down, accumulate_into=residual, ctx=ctx)
+
+
 class RoutedExperts(Part):
     """A mixture of clamped gated units: x += sum over the chosen experts e of s_e * expert_e(h), plus, if there is one, a
     shared expert for every row times sigmoid(Wsg h).
@@ -159,7 +195,8 @@ class RoutedExperts(Part):
     ``router`` "sigmoid": s = sigmoid(z), every expert by itself.  ``normalize``: the weights are the chosen experts' s divided
     by their sum (+ 1e-20).  ``route_scale`` multiplies the weights.  ``unit`` "gelu": an expert is Wd gelu(Wu h) with the exact
     gelu -- no gate matrix, no limit (``e<i>.{up,down}``, ``shared.{up,down}``).  ``shared_gate`` False: the shared expert is
-    added as it is (no ``shared.sg``)."""
+    added as it is (no ``shared.sg``).  ``router`` "chosen": the choice goes by the logits themselves (+ ``correction``), and the
+    weights are the softmax over the chosen logits alone.  ``router_bias``: ``router.b`` [experts] is added to the logits."""
     category = "feedforward"
     graph_safe = True     # launches kernels only: may run inside a captured graph
     accepts_lazy_norm = True
@@ -168,9 +205,13 @@ class RoutedExperts(Part):
     def __init__(self, hidden_size: int, experts: int, top: int, intermediate_size: int, limit: float = 0.0, groups: int = 1,
                  keep: int = 1, correction: bool = True, shared_size: int = 0, shared_limit: float = 0.0, slope: float = 1.702,
                  router: str = "softmax", normalize: bool = False, route_scale: float = 1.0, unit: str = "clamped_glu",
-                 shared_gate: bool = True):
-        if router not in ("softmax", "sigmoid") or unit not in ("clamped_glu", "gelu"):
-            raise ConfigError(f"routed experts: router {router!r} ('softmax' or 'sigmoid'), unit {unit!r} ('clamped_glu' or 'gelu')")
+                 shared_gate: bool = True, router_bias: bool = False):
+        if router not in ("softmax", "sigmoid", "chosen") or unit not in ("clamped_glu", "gelu"):
+            raise ConfigError(f"routed experts: router {router!r} ('softmax', 'sigmoid' or 'chosen'), unit {unit!r} "
+                              "('clamped_glu' or 'gelu')")
+        if router == "chosen" and normalize:
+            raise ConfigError("routed experts: a softmax over the chosen logits adds up to one: there is nothing to normalize")
+        self.over_chosen, self.router_bias = router == "chosen", bool(router_bias)
         self.squash, self.normalize, self.route_scale = router == "sigmoid", bool(normalize), float(route_scale)
         self.gated, self.shared_gate = unit == "clamped_glu", bool(shared_gate) and unit == "clamped_glu"
         self.hidden_size, self.experts, self.top, self.ff = int(hidden_size), int(experts), int(top), int(intermediate_size)
@@ -189,6 +230,8 @@ class RoutedExperts(Part):
         out = {"router": WeightSpec((self.experts, h))}
         if self.correction:
             out["correction"] = WeightSpec((self.experts,), kind="vector")
+        if self.router_bias:
+            out["router.b"] = WeightSpec((self.experts,), kind="vector")
         for name, size in [(f"e{e}", f) for e in range(self.experts)] + ([("shared", self.shared_ff)] if self.shared_ff else []):
             out.update({f"{name}.up": WeightSpec((size, h)), f"{name}.down": WeightSpec((h, size))})
             if self.gated:
@@ -208,6 +251,7 @@ class RoutedExperts(Part):
         self.w_route = ops.StreamedWeight(torch.cat([tensors["router"]] + ([tensors["shared.sg"]] if gated_shared else []),
                                                     dim=0).contiguous())
         self.correction_w = tensors["correction"].to(torch.float32).contiguous() if self.correction else None
+        self.router_b = tensors["router.b"].to(torch.float32).contiguous() if self.router_bias else None
         self.act_dtype = rt.act_dtype
 
     def step_work(self, batch, rows: int, elem: int):
@@ -228,18 +272,20 @@ class RoutedExperts(Part):
         E = self.experts
         z = linear(h, self.w_route, out_dtype=torch.float32)
         weights = ops.moe_route(z, E, self.top, self.groups, self.keep, self.correction_w, squash=self.squash,
-                                normalize=self.normalize, factor=self.route_scale)
+                                normalize=self.normalize, factor=self.route_scale, bias=self.router_b,
+                                over_chosen=self.over_chosen)
         gu = linear(h, self.w_gu, out_dtype=self.act_dtype)
         if not self.gated:
             linear(ops.routed_gelu(gu, weights, E, self.ff, self.shared_ff, out=gu), self.w_down, accumulate_into=residual, ctx=ctx)
             return
         y = ops.routed_glu(gu, weights, E, self.ff, self.limit, shared_ff=self.shared_ff, shared_limit=self.shared_limit,
-                           shared_logit=z[:, E:E + 1] if self.shared_ff else None, slope=self.slope)
+                           shared_logit=z[:, E:E + 1] if self.shared_ff and self.shared_gate else None, slope=self.slope)
         linear(y, self.w_down, accumulate_into=residual, ctx=ctx)
 
 
 register_part("feedforward", "swiglu", SwiGLU)
 register_part("feedforward", "dense_gelu", DenseGELU)
+register_part("feedforward", "dense_squared_relu", DenseSquaredReLU)
 register_part("feedforward", "routed_experts", RoutedExperts)
 register_part("feedforward", "clamped_glu", ClampedGLU)
 register_part("feedforward", "dense_xielu", DenseXIELU)

@@ -22,13 +22,18 @@ class LatentAttention(Part):
 
     Only c and kr are cached (cache.specs.PagedLatent).  The keys' up-projection is absorbed into the query
     (Wuk_a^T q_plain scores against c directly) and the values' up-projection is applied to the weighted sum of the
-    latents, so no key or value is ever made per head and token; scores, weights and the sums are float32."""
+    latents, so no key or value is ever made per head and token; scores, weights and the sums are float32.
+
+    ``borrows``: the layer makes no latent (no ``dkv``, no ``dkv.norm``) -- it reads the cache rows another layer of the
+    same kv_rank and rot_dim writes, with queries, up-projections, window and sink of its own.  Which one is the
+    schedule's business (the entry names that layer's cache stream and does not write)."""
     category = "mixer"
     graph_safe = True     # launches kernels only: may run inside a captured graph
     adds_one_product = True   # the output is one last product through linear(): a block may hand it ops.Fresh
+    accepts_lazy_norm = True  # (one product reads the norm)
 
-    def __init__(self, hidden_size: int, heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, scale: float,
-                 rot_dims: int, rot_base: float, eps: float, sink: bool = True, window: int = 0):
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, kv_rank: int, scale: float, eps: float, rot_dim: int = 0,
+                 rot_dims: int = 0, rot_base: float = 10000.0, sink: bool = True, window: int = 0, borrows: bool = False):
         for name, v in (("heads", heads), ("dim", dim), ("vdim", vdim), ("kv_rank", kv_rank), ("hidden_size", hidden_size)):
             if int(v) <= 0:
                 raise ConfigError(f"latent attention: {name} must be positive, got {v}")
@@ -41,16 +46,18 @@ class LatentAttention(Part):
         self.hidden_size, self.heads, self.dim, self.rot_dim = int(hidden_size), int(heads), int(dim), int(rot_dim)
         self.vdim, self.kv_rank, self.scale, self.rot_dims = int(vdim), int(kv_rank), float(scale), int(rot_dims)
         self.rot_base, self.eps, self.sink, self.window = float(rot_base), float(eps), bool(sink), int(window)
+        self.borrows = bool(borrows)
 
     def cache_spec(self):
         return PagedLatent(self.kv_rank, self.rot_dim, self.window)
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
         H, w = self.heads, self.hidden_size
-        out = {"q": WeightSpec((H * (self.dim + self.rot_dim), w)), "dkv": WeightSpec((self.kv_rank + self.rot_dim, w)),
-               "dkv.norm": WeightSpec((self.kv_rank,), kind="vector", init="ones"),
-               "uk": WeightSpec((H * self.dim, self.kv_rank)), "uv": WeightSpec((H * self.vdim, self.kv_rank)),
-               "o": WeightSpec((w, H * self.vdim))}
+        out = {"q": WeightSpec((H * (self.dim + self.rot_dim), w))}
+        if not self.borrows:
+            out.update({"dkv": WeightSpec((self.kv_rank + self.rot_dim, w)), "dkv.norm": WeightSpec((self.kv_rank,), kind="vector", init="ones")})
+        out.update({"uk": WeightSpec((H * self.dim, self.kv_rank)), "uv": WeightSpec((H * self.vdim, self.kv_rank)),
+                    "o": WeightSpec((w, H * self.vdim))})
         if self.sink:
             out["sink"] = WeightSpec((H,), kind="vector")
         return out
@@ -58,9 +65,9 @@ class LatentAttention(Part):
     def bind(self, tensors, rt) -> None:
         H = self.heads
         # one product for the queries and the latent: their rows one after the other
-        self.w_qd = ops.StreamedWeight(torch.cat([tensors["q"], tensors["dkv"]], dim=0).contiguous())
+        self.w_qd = ops.StreamedWeight(tensors["q"] if self.borrows else torch.cat([tensors["q"], tensors["dkv"]], dim=0).contiguous())
         self.w_o = ops.StreamedWeight(tensors["o"])
-        self.g = tensors["dkv.norm"].to(torch.float32).contiguous()
+        self.g = None if self.borrows else tensors["dkv.norm"].to(torch.float32).contiguous()
         # [heads, rank, dim]: the keys' up-projection as it is applied to the query
         self.uk_t = tensors["uk"].view(H, self.dim, self.kv_rank).transpose(1, 2).contiguous()
         self.uv = tensors["uv"].view(H, self.vdim, self.kv_rank).contiguous()
@@ -77,11 +84,19 @@ class LatentAttention(Part):
         return (super().working_bytes_per_row(elem) + 4 * self.heads * (2 * self.kv_rank + self.rot_dim)
                 + self.heads * self.vdim * elem)
 
+    def wants_prepared_norm(self, n_rows: int) -> bool:
+        """Whether the first product is better served by a norm that the product before prepared than by fusing the
+        norm or running it: the weight's own plan says (ops.LinearPlan.wants_prepared)."""
+        return self.act_dtype == torch.bfloat16 and self.w_qd.plan.wants_prepared(n_rows)
+
     def forward(self, h, ctx, cache, residual, writes: bool = True) -> None:
-        H, rank, rot, t = self.heads, self.kv_rank, self.rot_dim, h.shape[0]
+        H, rank, rot = self.heads, self.kv_rank, self.rot_dim
+        if self.borrows and writes:
+            raise ConfigError("latent attention: a layer without a latent of its own cannot write a cache stream")
         n_q = H * (self.dim + rot)
         qd = linear(h, self.w_qd, out_dtype=self.act_dtype)
-        q, dkv = qd[:, :n_q], qd[:, n_q:]
+        t = qd.shape[0]
+        q, dkv = qd[:, :n_q], None if self.borrows else qd[:, n_q:]
         q_lat = torch.empty((t, H, rank + rot), dtype=torch.float32, device=q.device)
         angles = None
         if self.rot_dims:                 # the same in every layer that rotates alike: a table made once a step

@@ -69,6 +69,24 @@ def linear(x: Union[torch.Tensor, Normed], w, out_dtype: Optional[torch.dtype] =
     return ops.gemm_generic(x, w, out_dtype, accumulate_into)
 
 
+def linear_squared_relu(x: Union[torch.Tensor, Normed], w, out_dtype: torch.dtype) -> torch.Tensor:
+    """max(x W^T, 0)^2: applied to the float sums inside the product's kernel where a matrix-core kernel takes the
+    operands (with the norm fused or prepared like any product's), else by a kernel behind it."""
+    if isinstance(x, Normed):
+        if out_dtype == torch.bfloat16:
+            fused = _prepared_norm(x, w, ops.EPI_SQUARED_RELU)
+            if fused is None:
+                fused = _fused_norm(x, w, ops.EPI_SQUARED_RELU)
+            if fused is not None:
+                return fused
+        x = x.tensor()
+    fast = ops.gemm_fast(x, w, out_dtype, squared_relu=True)
+    if fast is not None:
+        return fast
+    z = linear(x, w, out_dtype=out_dtype)
+    return ops.squared_relu(z, out=z)
+
+
 def linear_swiglu(x: Union[torch.Tensor, Normed], w_gate_up, interleaved: bool = False) -> torch.Tensor:
     """silu(x Wg^T) * (x Wu^T) for w_gate_up = gate rows followed by up rows, or (interleaved)
     blocks of eight gate rows and the eight up rows of the same outputs."""
