@@ -149,6 +149,29 @@ LAGUSUN_SIZES = {
     "2k": (lagusun_shape(2048, 5, 16, 4, 64, 128, 8, 2, 2688), MILENEX_SIZES["2k"][0]),
     "4k": (lagusun_shape(4096, 5, 32, 8, 64, 128, 8, 2, 4800), MILENEX_SIZES["4k"][0]),
 }
+
+
+def baselix_shape(width, layers, heads, dim, vdim, kv_rank, ff, experts, top, expert_ff, window=1024, vocab=32000):
+    """A Baselix configuration of real layer sizes: layers in pairs, the second of which reads the first one's latents; the
+    first of a pair with a dense squared-relu feed-forward, the second with ``top`` of ``experts`` routed clamped units and
+    a shared one."""
+    dense = dict(kind="dense", ff=ff)
+    moe = dict(kind="moe", expert=dict(ff=expert_ff, limit=7.0), router=dict(experts=experts, top=top), shared=dict(ff=expert_ff, limit=7.0))
+    mixer = dict(heads=heads, dim=dim, vdim=vdim, kv_rank=kv_rank, scale=dim ** -0.5, mask=dict(size=window))
+    order = [dict(type="latent_attention", mixer=dict(mixer, kv_from=i - 1) if i % 2 else dict(mixer), mlp=moe if i % 2 else dense)
+             for i in range(layers)]
+    return dict(architecture="Baselix", vocab=vocab, width=width, max_positions=8192, norm=dict(eps=1e-6), residual_mult=0.25,
+                logit_softcap=30.0, layers=order)
+
+
+# --only baselix: the design at a few sizes that resemble a real model's layers, each beside the Mamenex decoder (the
+# other design here with latent attention and a dense feed-forward) and the Milenex decoder (the other one with clamped
+# routed experts) of the same width, number of layer runs and head count.
+BASELIX_SIZES = {
+    "1k": (baselix_shape(1024, 6, 8, 64, 64, 256, 4096, 8, 2, 896), MAMENEX_SIZES["1k"][0], MILENEX_SIZES["1k"][0]),
+    "2k": (baselix_shape(2048, 6, 16, 128, 128, 512, 8192, 8, 2, 1792), MAMENEX_SIZES["2k"][0], MILENEX_SIZES["2k"][0]),
+    "4k": (baselix_shape(4096, 6, 32, 128, 128, 512, 14336, 8, 2, 3200), MAMENEX_SIZES["4k"][0], MILENEX_SIZES["4k"][0]),
+}
 BASELINE_DECODE_B1 = 77.3                   # the reference's only FP16 decode number (batch 1, RTX 3050)
 
 
@@ -321,7 +344,8 @@ def kernel_table(model, cfg, prefill_tokens, batch, context, dtype):
 
 def run_mamenex(size, args, only="mamenex", names=("mamenex", "llama"), sizes=None):
     """Prefill and decode of a design at one size beside another decoder of equal size (Mamenex beside Llama, Nagezen
-    beside Mamenex, Milenex beside Nagezen, Lagusun beside Milenex); with --kernels the per-kernel tables of both."""
+    beside Mamenex, Milenex beside Nagezen, Lagusun beside Milenex, Baselix beside Mamenex and Milenex); with --kernels the
+    per-kernel tables of all."""
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     elem = 2 if args.dtype == "bf16" else 4
     line = {"only": only, "size": size, "dtype": args.dtype, "prefill_tokens": args.prefill_tokens, "batch": args.batch,
@@ -489,9 +513,9 @@ def main() -> int:
     ap.add_argument("--top-p", type=float, default=1.0, help="--only serve: ... and this top-p (1: none)")
     ap.add_argument("--gather-ms", type=float, default=0.0,
                     help="--only chat: the scheduler waits this long before it admits those who came while others decode")
-    ap.add_argument("--sizes", default="1k,2k,4k", help="--only mamenex, nagezen, milenex, lagusun: which of the sizes " + ", ".join(MAMENEX_SIZES))
-    ap.add_argument("--kernels", action="store_true", help="--only mamenex, nagezen, milenex, lagusun: add the per-kernel tables (time, part of the roofline)")
-    ap.add_argument("--only", choices=["decode", "prefill", "serve", "chat", "gemm", "peaks", "mamenex", "nagezen", "milenex", "lagusun"], default=None,
+    ap.add_argument("--sizes", default="1k,2k,4k", help="--only mamenex, nagezen, milenex, lagusun, baselix: which of the sizes " + ", ".join(MAMENEX_SIZES))
+    ap.add_argument("--kernels", action="store_true", help="--only mamenex, nagezen, milenex, lagusun, baselix: add the per-kernel tables (time, part of the roofline)")
+    ap.add_argument("--only", choices=["decode", "prefill", "serve", "chat", "gemm", "peaks", "mamenex", "nagezen", "milenex", "lagusun", "baselix"], default=None,
                     help="run one part only and print its own short line (for profiling); peaks: what a kernel that only "
                          "reads, and one of nothing but matrix-core instructions, reach on this device")
     ap.add_argument("--mnk", default="2048,11264,2048",
@@ -523,6 +547,10 @@ def main() -> int:
     if args.only == "lagusun":
         for size in args.sizes.split(","):
             print(json.dumps(run_mamenex(size, args, "lagusun", ("lagusun", "milenex"), LAGUSUN_SIZES)), flush=True)
+        return 0
+    if args.only == "baselix":
+        for size in args.sizes.split(","):
+            print(json.dumps(run_mamenex(size, args, "baselix", ("baselix", "mamenex", "milenex"), BASELIX_SIZES)), flush=True)
         return 0
     from bare_cuda_4gib_amd.csrc.peaks import measured_peaks
     measured = measured_peaks()
