@@ -43,6 +43,9 @@ inline std::vector<double> gemm(const std::vector<double>& a, const std::vector<
   return out;
 }
 
+// max(z, 0)^2
+inline double squared_relu(double z) { return z > 0.0 ? z * z : 0.0; }
+
 // silu(g) * u, silu(g) = g / (1 + exp(-g)) (reference: engine/kernels/swiglu.cu:22-23).
 inline double swiglu(double g, double u) { return g / (1.0 + std::exp(-g)) * u; }
 

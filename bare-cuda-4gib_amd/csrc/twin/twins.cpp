@@ -50,6 +50,20 @@ bool embed() {
     RUN(bc4g_embed_rows(dtype ? static_cast<const void*>(t16.p) : t32.p, dtype, di.p, out.p, n, hidden, vocab, factor, 1, kStream));
     for (double& v : want) v *= 2.0 * factor;
     ok &= close(dtype ? "scaled rows of a bfloat16 table" : "scaled rows of a float table", widen(out.get()), want, 1e-6, 0.0);
+    // the same rows plus a row for every position, times a factor, stored and then added to what is there
+    const int n_places = 9;
+    const std::vector<float> place_rows = normals(rng, static_cast<size_t>(n_places) * hidden);
+    const std::vector<int32_t> positions = {0, 8, 3, 3, 1, 7, 2};
+    const std::vector<double> places = dtype ? widen(as_bf16(place_rows)) : widen(place_rows);
+    Dev<float> p32(place_rows);
+    Dev<bf16> p16(as_bf16(place_rows));
+    Dev<int32_t> dpos(positions);
+    for (int add = 0; add < 2; ++add)
+      RUN(bc4g_embed_placed(dtype ? static_cast<const void*>(t16.p) : t32.p, dtype ? static_cast<const void*>(p16.p) : p32.p, dtype, di.p,
+                            dpos.p, out.p, n, hidden, vocab, n_places, factor, add, kStream));
+    for (int r = 0; r < n; ++r)
+      for (int c = 0; c < hidden; ++c) want[static_cast<size_t>(r) * hidden + c] += 2.0 * factor * places[static_cast<size_t>(positions[r]) * hidden + c];
+    ok &= close(dtype ? "placed rows of a bfloat16 table" : "placed rows of a float table", widen(out.get()), want, 1e-6, 1e-6);
   }
   return ok;
 }
@@ -168,6 +182,10 @@ bool gemm_skinny() {
     RUN(bc4g_gemm_skinny(dx.p, packed.p, acc.p, 2, m, n, k, kStream));
     RUN(bc4g_gemm_skinny(dx.p, packed.p, act.p, 3, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, 6, m, n, k, kStream));
+    std::vector<double> squared = want;
+    for (double& v : squared) v = plain::squared_relu(v);
+    ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
     ok &= close("float out", widen(o32.get()), want, 1e-4, 1e-4);
     std::vector<double> sum = want, gated;
     for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i];
@@ -259,6 +277,10 @@ bool gemm_mfma() {
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, acc.p, 2, m, n, k, kStream));
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, act.p, 3, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, 6, m, n, k, kStream));
+    std::vector<double> squared = want;
+    for (double& v : squared) v = plain::squared_relu(v);
+    ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
     ok &= close("float out", widen(o32.get()), want, 1e-4, 1e-4);
     std::vector<double> sum = want, gated;
     for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i];
