@@ -9,3 +9,4 @@ from .nagezen import NagezenConfig  # noqa: F401
 from .milenex import MilenexConfig  # noqa: F401
 from .lagusun import LagusunConfig  # noqa: F401
 from .baselix import BaselixConfig  # noqa: F401
+from .varolix import VarolixConfig  # noqa: F401

@@ -42,20 +42,20 @@ int bc4g_stream_update(float* x, const float* y, const float* scale, const float
 int bc4g_embed_beside(const float* x, const void* table, int table_dtype, const int32_t* ids, float factor, void* out,
                       int out_dtype, int n_tokens, int hidden, int vocab, void* stream);
 // The same for a stream whose last addition is still in parts [n_parts, n_rows, hidden] (float32, as
-// bc4g_gemm_mfma_parts leaves them): x += parts[0] + parts[1] + ... in that order, written back, then out = its norm
-// (bfloat16).  hidden a multiple of 8, at most 8192.
-int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const void* w, int w_dtype, void* out, int out_dtype,
+// bc4g_gemm_mfma_parts leaves them): x += bias (a number a column, null: none) + parts[0] + parts[1] + ... in that order,
+// written back, then out = its norm (bfloat16).  hidden a multiple of 8, at most 8192.
+int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const float* bias, const void* w, int w_dtype, void* out, int out_dtype,
                      int n_rows, int hidden, float eps, void* stream);
 
 // out[m, n] (+)= sum_k a[m, k] * w[n, k]        (gemm_tiled.cuh:36-96, plain float FMA)
-// accumulate != 0 adds into a float `out` (the residual stream).
+// accumulate != 0 adds into a float `out` (the residual stream), and with it bias [n] (null: none).
 int bc4g_gemm_generic(const void* a, int a_dtype, const void* w, int w_dtype, void* out,
-                      int out_dtype, int accumulate, int m, int n, int k, void* stream);
+                      int out_dtype, int accumulate, const float* bias, int m, int n, int k, void* stream);
 
 // out[t, i] = silu(gate_i) * up_i                                        (swiglu.cu:17-25)
 // interleaved 0: gu[t] = all gates, then all ups.  1: blocks of 16 = eight gates, then the eight
-// ups of the same outputs.
-int bc4g_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int interleaved, void* stream);
+// ups of the same outputs.  act 1: the gelu written with tanh instead of the silu.
+int bc4g_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int interleaved, int act, void* stream);
 
 // Rotates q (in place) and k by each row's position, and writes k and v into
 // their cache pages (rope.cu:18-55, kv_cache_write.cu:10-20).
@@ -124,8 +124,9 @@ extern "C" {
 // of a k-step holds row l % 16 of the block and k 8 * (l / 16) .. + 7 of the step, zeros past n and k.
 // epilogue: 0 store bfloat16 [m, n]; 1 store float32; 2 add into float32;
 // 3 SwiGLU: every 16 rows of w are eight gate rows and the eight up rows of the same outputs
-// (n = 2 * inter), out bfloat16 [m, inter] = silu(gate) * up; 6 store max(sum, 0)^2 as bfloat16 [m, n].
-int bc4g_gemm_skinny(const void* x, const void* w, void* out, int epilogue, int m, int n, int k, void* stream);
+// (n = 2 * inter), out bfloat16 [m, inter] = silu(gate) * up; 6 store max(sum, 0)^2 as bfloat16 [m, n]; 7 as 3 with
+// the gelu written with tanh for the silu.  bias [n] (float32; null: none) joins the sums of epilogue 2.
+int bc4g_gemm_skinny(const void* x, const void* w, void* out, const float* bias, int epilogue, int m, int n, int k, void* stream);
 }
 
 extern "C" {
@@ -162,24 +163,24 @@ int bc4g_attention_mfma(const void* qkv, int q_stride, void* out, float* part_o,
 extern "C" {
 // bfloat16 a [m, k] times bfloat16 w [n, k] transposed on the matrix cores, any m.
 // epilogue: 0 store bfloat16; 1 store float32; 2 add into float32; 3 SwiGLU as in bc4g_gemm_skinny; 6 store
-// max(sum, 0)^2 as bfloat16.
+// max(sum, 0)^2 as bfloat16; 7 as 3 with the gelu written with tanh.  bias [n] (null: none) joins the sums of epilogue 2.
 // w_packed 1: w lies in the order of the weight-streaming kernel (bc4g_gemm_skinny: [ceil(n / 16)][k / 32][64 lanes][8]),
 // so that one copy of a weight serves both kernels: the kernel with operands straight into LDS reads it (k a multiple
 // of 64, operands on 16-byte boundaries).  0: w lies by rows, [n, k], for the kernel that stages its tiles through
 // registers (any k that is a multiple of 8).  The sums are the same bits either way.  The three entry points below
 // are forms of the first kernel and take the packed weight only.
-int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* out, int epilogue, int m, int n, int k, void* stream);
+int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* out, const float* bias, int epilogue, int m, int n, int k, void* stream);
 // The same product with k cut into k_parts equal parts (each a multiple of 64), part p's sums stored as float32 in
 // parts [k_parts, m, n]: for few rows and a long k, where one workgroup per 64 x 64 tile would walk all of k alone.
 // Whoever reads the parts adds them up in order (bc4g_rmsnorm_sum).
 int bc4g_gemm_mfma_parts(const void* a, const void* w, int w_packed, float* parts, int m, int n, int k, int k_parts,
                          void* stream);
-// The SwiGLU product (epilogue 3) of rows that lack their RMSNorm's common factor: a = bfloat16(residual * g) [m, k] and
+// The SwiGLU product (epilogue 3; gelu 1: epilogue 7) of rows that lack their RMSNorm's common factor: a = bfloat16(residual * g) [m, k] and
 // the parts of the rows' sums of squares as bc4g_gemm_skinny_emit leaves them (ssq_parts [ssq_blocks][ssq_stride]); every
 // row's sums are multiplied by 1 / sqrt(sum of squares / k + eps) before the activation, the parts added in the order
 // of bc4g_gemm_skinny_prenormed.  k a multiple of 64, n of 16, operands on 16-byte boundaries; any m.
 int bc4g_gemm_mfma_swiglu_scaled(const void* a, const float* ssq_parts, int ssq_blocks, int ssq_stride, float eps,
-                                 const void* w, int w_packed, void* out, int m, int n, int k, void* stream);
+                                 const void* w, int w_packed, void* out, int gelu, int m, int n, int k, void* stream);
 // The output tile (rows, columns) bc4g_gemm_mfma (qkv 0) or bc4g_gemm_mfma_qkv (qkv 1) takes for these operands: for
 // the accounting of bytes and for tests that want to meet every tile.  Launches nothing.
 int bc4g_gemm_mfma_tile(const void* a, const void* w, int m, int n, int k, int qkv, int* rows, int* cols);
@@ -219,12 +220,12 @@ int bc4g_gemm_skinny_qkv(const void* x, const void* g, int g_dtype, float eps, c
 
 extern "C" {
 // The adding product that prepares the RMSNorm after it: out (the float32 residual stream, [m, n])
-// += x w^T; emit_x [m, n] = bfloat16(new residual * g) (g: that norm's scale, g_dtype 0 float32, 1
+// += x w^T + bias (null: none); emit_x [m, n] = bfloat16(new residual * g) (g: that norm's scale, g_dtype 0 float32, 1
 // bfloat16); emit_ssq [ceil(n / 16)][emit_stride]: block b's part (16 columns) of every row's sum of
 // squares.  bc4g_gemm_skinny_prenormed takes such an x (k = this n) and the parts instead of a norm:
 // out = rmsnorm(residual) w^T, the row's rsqrt(sum of the parts / k + eps) applied to the finished
 // sums; epilogues of bc4g_gemm_skinny except the adding one.
-int bc4g_gemm_skinny_emit(const void* x, const void* w, float* out, const void* g, int g_dtype, void* emit_x,
+int bc4g_gemm_skinny_emit(const void* x, const void* w, float* out, const float* bias, const void* g, int g_dtype, void* emit_x,
                           float* emit_ssq, int emit_stride, int m, int n, int k, void* stream);
 int bc4g_gemm_skinny_prenormed(const void* x, const float* ssq_parts, int ssq_blocks, int ssq_stride, float eps,
                                const void* w, void* out, int epilogue, int m, int n, int k, void* stream);
@@ -286,14 +287,18 @@ int bc4g_rglru_scan(const float* pre, const void* u, const void* y, int dtype, c
 // (bc4g_latent_angles makes it, the angles worked out in double: once a step for all layers of one rotation).  q_row,
 // dkv_row: elements from one row to the next (q and dkv may be parts of one product's rows).  Without a cache (a layer
 // that reads another one's latents) only the queries are rotated and dkv, g and slot_map may be null; with rot 0 only
-// the cache row is written and q and q_lat may be null.
+// the cache row is written and q and q_lat may be null (as they may where the queries do not exist yet).  halves 1: element
+// i of the first dims turns with element i + dims / 2 instead.  low [T, low_rank] (null: none; rows low_row apart): a latent
+// of the queries' own, written to low_out [T, low_rank] as rmsnorm(low) * low_g with the same eps.
 int bc4g_latent_angles(const int32_t* positions, float* table, int n_rows, int dims, float base, void* stream);
 int bc4g_latent_prepare(const void* q, const void* dkv, int dtype, const float* g, float eps, const float* angles,
                         const int32_t* slot_map, void* cache, float* q_lat, int n_rows, int heads, int plain, int rot,
-                        int rank, int dims, long q_row, long dkv_row, void* stream);
-// out[t, h, :n] = w[h] a[t, h, :k] for every head: a at a + t * a_row + h * a_head, out likewise, w [heads, n, k].
+                        int rank, int dims, long q_row, long dkv_row, int halves, const void* low, const float* low_g, void* low_out,
+                        int low_rank, long low_row, void* stream);
+// out[t, h, :n] = w[h] a[t, h, :k] for every head: a at a + t * a_row + h * a_head, out likewise, w [heads, n, k].  gate
+// [T, heads] (null: none; rows gate_row apart): head h's outputs are multiplied by sigmoid(gate[t, h]).
 int bc4g_heads_gemm(const void* a, int a_dtype, long a_row, long a_head, const void* w, int w_dtype, void* out, int out_dtype,
-                    long o_row, long o_head, int m, int n, int k, int heads, void* stream);
+                    long o_row, long o_head, int m, int n, int k, int heads, const void* gate, int gate_dtype, long gate_row, void* stream);
 // out[t, h, :rank] = sum_j p_j cache[j, :rank] with p = exp(scale * q_lat[t, h] . cache[j]) over the keys the row sees
 // (max(0, p - window + 1) .. p), divided by their sum plus exp(sink[h]) (sink null: no such term).  float32 in and out.
 int bc4g_attention_latent(const float* q_lat, float* out, const void* cache, int dtype, const float* sink,
@@ -344,6 +349,10 @@ struct bc4g_prepare_section {
   // norm_rows 1: the norm before the rotation is taken over the whole row -- all heads at once, mean over heads * dim --
   // and norm_w is [heads * dim]; 0: over each head, norm_w [dim].
   int pairing, unit_after, norm_rows;
+  // positions (null: none): the head is multiplied, last, by 1 + temp_coef ln(floor((positions[row] + 1) / temp_every) + 1).
+  float temp_coef;
+  double temp_every;
+  const int32_t* positions;
 };
 int bc4g_heads_prepare_many(const bc4g_prepare_section* sections, int n_sections, int n_rows, void* stream);
 int bc4g_heads_prepare(const void* in, int in_dtype, long in_row, const float* bias, const float* norm_w, float eps,
@@ -365,6 +374,21 @@ int bc4g_decay_scan(const void* q, int q_dtype, long q_row, float q_scale, const
                     const int32_t* seq_start, const int32_t* seq_slots, const int32_t* chunk_base, int n_rows, int n_seqs,
                     int most_rows, int heads, int dim, int vdim, void* stream);
 
+// A matrix memory per head with exponential input gates and a normaliser (matrix_memory.hip): along every request's rows
+//   m_t = max(f_t + m_(t-1), i_t),  S_t = e^(f_t + m_(t-1) - m_t) S_(t-1) + e^(i_t - m_t) k_t v_t^T,  n_t likewise with k_t,
+//   o_t = S_t^T (q_t q_scale) / (max(|n_t . q_t q_scale|, e^(-m_t)) + 1e-6),
+//   out = o_t / sqrt(mean(o_t^2) + eps) * weight * sigmoid(gate) * factor      per head, [T, heads * vdim], rows out_row apart
+// with i = cap tanh((zi + bi) / cap), f = log sigmoid(cap tanh((zf + bf) / cap)).  q, k [T, heads * dim], v, gate
+// [T, heads * vdim], zi, zf [T, heads] are parts of rows `row` elements apart, of one dtype.  State float32: S [slots, heads, dim,
+// vdim], n [slots, heads, dim], m [slots, heads], read and left in every request's slot.  Requests that bring more than 32
+// rows need scratch: gates [3, T, heads], chunk_S [chunks, heads, dim, vdim], chunk_n [chunks, heads, dim], chunk_decay
+// [chunks, heads] and chunk_base as bc4g_decay_scan.  dim and vdim at most 256.
+int bc4g_matrix_memory(const void* q, const void* k, const void* v, const void* gate, const void* zi, const void* zf, int dtype,
+                       long row, const float* bi, const float* bf, float cap, float q_scale, const float* weight, float eps,
+                       float factor, void* out, int out_dtype, long out_row, float* S, float* n, float* m, float* gates,
+                       float* chunk_S, float* chunk_n, float* chunk_decay, const int32_t* seq_start, const int32_t* seq_slots,
+                       const int32_t* chunk_base, int n_rows, int n_seqs, int most_rows, int heads, int dim, int vdim, void* stream);
+
 // Attention with one or two score maps per query head over the same values (attention_maps.hip): q float32
 // [T, heads, maps, dim]; keys [page, kv_head * maps + map, token, dim], values [page, kv_head, token, vdim]; a row at p
 // sees j <= p with p - j < window or j < keep_first (window 0: all).  o = a1 - lambda a2 (one map: a1), with normalize
@@ -374,10 +398,11 @@ int bc4g_decay_scan(const void* q, int q_dtype, long q_row, float q_scale, const
 // block > 0 (then window and keep_first 0): a row sees the keys of its own block of `block` positions counted from 0,
 // j <= p with j / block == p / block.  cap > 0: the scaled score becomes cap tanh(score / cap).  point [heads] (or null; then
 // no sink): no softmax -- the weight of a visible key is sigmoid(score + point[head]), nothing is normalised over keys.
+// out's rows lie out_row elements apart (it may be a part of wider rows).
 int bc4g_attention_maps(const float* q, long q_row, const void* k_cache, const void* v_cache, int cache_dtype,
                         const int32_t* block_table, int table_stride, const int32_t* row_seq, const int32_t* positions,
                         float lambda, int normalize, float eps, float factor, const void* gate, int gate_dtype, long gate_row,
-                        int gate_act, void* out, int out_dtype, int n_rows, int n_heads, int n_kv_heads, int maps, int dim,
+                        int gate_act, void* out, int out_dtype, long out_row, int n_rows, int n_heads, int n_kv_heads, int maps, int dim,
                         int vdim, int page_tokens, int window, int keep_first, float scale, int waves, const float* sink,
                         const float* far1, const float* far2, int block, float cap, const float* point, void* stream);
 

@@ -7,8 +7,9 @@
 // decoded tokens are the same to these kernels.
 //
 //   bc4g_latent_prepare     norms the latent, rotates the shared key part and writes both into the row's cache
-//                           slot; rotates every head's rotated query part into the absorbed query
-//   bc4g_heads_gemm         out[t, h, :] = w[h] a[t, h, :] for every head (both up-projections)
+//                           slot; rotates every head's rotated query part into the absorbed query; norms the
+//                           queries' own latent, where they have one
+//   bc4g_heads_gemm         out[t, h, :] = w[h] a[t, h, :] for every head (both up-projections), times a gate a head
 //   bc4g_attention_latent   the attention itself, over the paged cache
 #include <float.h>
 #include <math.h>
@@ -47,18 +48,55 @@ __global__ void latent_angles_kernel(const int32_t* __restrict__ positions, floa
 // One workgroup a row.  q: [T, heads, plain + rot] (as projected); dkv: [T, rank + rot] (rows q_row and dkv_row elements
 // apart: both may be parts of one product's rows); q_lat: [T, heads, rank + rot]
 // float, of which this kernel writes the last rot of every head; the row's cache slot receives [normed latent | rotated
-// key part].  Neighbouring elements 2i and 2i + 1 of the first `dims` of a rotated part are a pair; the rest passes.
+// key part].  Elements 2i and 2i + 1 of the first `dims` of a rotated part are a pair, or with halves element i and
+// element i + dims / 2; the rest passes.  low [T, low_rank] (rows low_row apart): the queries' latent, which goes to
+// low_out [T, low_rank] normed with the weight low_g.
+struct PairOf {
+  int other, angle;      // the pair's other member, and the pair's number
+  bool second;           // whether this element is the pair's second member
+};
+__device__ inline PairOf pair_of(int i, int dims, int halves) {
+  if (!halves) return PairOf{i ^ 1, i / 2, (i & 1) != 0};
+  const int half = dims / 2;
+  return i < half ? PairOf{i + half, i, false} : PairOf{i - half, i - half, true};
+}
+
+struct LowQuery {
+  const void* low;
+  const float* g;
+  void* out;
+  long row;
+  int rank;
+};
+
 template <typename T>
 __global__ __launch_bounds__(kPrepBlock) void latent_prepare_kernel(
     const T* __restrict__ q, const T* __restrict__ dkv, const float* __restrict__ g, float eps,
     const float* __restrict__ angles, const int32_t* __restrict__ slot_map, T* __restrict__ cache,
-    float* __restrict__ q_lat, int heads, int plain, int rot, int rank, int dims, long q_row, long dkv_row, int first_part) {
+    float* __restrict__ q_lat, int heads, int plain, int rot, int rank, int dims, long q_row, long dkv_row, int parts, int halves,
+    const LowQuery lq) {
   __shared__ float scratch[16];
   extern __shared__ float cs[];                     // [dims / 2][2]: the row's cosines and sines
   const long row = blockIdx.x;
   for (int i = threadIdx.x; i < dims; i += kPrepBlock) cs[i] = angles[row * dims + i];
-  // (two workgroups a row, as far as there is work for them: part 0 norms and stores the cache row, part 1 rotates the queries)
-  if (static_cast<int>(blockIdx.y) + first_part == 1) {
+  // (a workgroup a row for each part there is work for: part 0 norms and stores the cache row, part 1 rotates the queries,
+  // part 2 norms the queries' latent; blockIdx.y counts the parts that are there)
+  int part_no = 0;
+  for (int left = blockIdx.y;; ++part_no)
+    if ((parts >> part_no & 1) && left-- == 0) break;
+  if (part_no == 2) {
+    const T* lo = static_cast<const T*>(lq.low) + row * lq.row;
+    T* to = static_cast<T*>(lq.out) + row * lq.rank;
+    float sum = 0.f;
+    for (int i = threadIdx.x; i < lq.rank; i += kPrepBlock) {
+      const float v = to_float(lo[i]);
+      sum += v * v;
+    }
+    const float by = 1.0f / sqrtf(block_sum(sum, scratch) / static_cast<float>(lq.rank) + eps);
+    for (int i = threadIdx.x; i < lq.rank; i += kPrepBlock) to[i] = from_float<T>(to_float(lo[i]) * by * lq.g[i]);
+    return;
+  }
+  if (part_no == 1) {
     __syncthreads();
     const T* qr = q + row * q_row;
     float* ql = q_lat + row * heads * (rank + rot);
@@ -67,8 +105,9 @@ __global__ __launch_bounds__(kPrepBlock) void latent_prepare_kernel(
       const T* part = qr + h * (plain + rot) + plain;
       float v = to_float(part[i]);
       if (i < dims) {
-        const float c = cs[2 * (i / 2)], s = cs[2 * (i / 2) + 1], other = to_float(part[i ^ 1]);
-        v = (i & 1) ? v * c + other * s : v * c - other * s;
+        const PairOf p = pair_of(i, dims, halves);
+        const float c = cs[2 * p.angle], s = cs[2 * p.angle + 1], other = to_float(part[p.other]);
+        v = p.second ? v * c + other * s : v * c - other * s;
       }
       ql[h * (rank + rot) + rank + i] = v;
     }
@@ -87,13 +126,26 @@ __global__ __launch_bounds__(kPrepBlock) void latent_prepare_kernel(
     for (int i = threadIdx.x; i < rot; i += kPrepBlock) {
       float v = to_float(lat[rank + i]);
       if (i < dims) {
-        const float c = cs[2 * (i / 2)], s = cs[2 * (i / 2) + 1], other = to_float(lat[rank + (i ^ 1)]);
-        v = (i & 1) ? v * c + other * s : v * c - other * s;
+        const PairOf p = pair_of(i, dims, halves);
+        const float c = cs[2 * p.angle], s = cs[2 * p.angle + 1], other = to_float(lat[rank + p.other]);
+        v = p.second ? v * c + other * s : v * c - other * s;
       }
       to[rank + i] = from_float<T>(v);
     }
   }
 }
+
+// A product's head gate: a number a row and head, of which the sigmoid multiplies the head's outputs (none: 1).
+struct HeadGate {
+  const void* z;
+  long row;
+  int dtype;
+  __device__ float of(long r, int h) const {
+    if (!z) return 1.0f;
+    const float v = dtype == kF32 ? static_cast<const float*>(z)[r * row + h] : to_float(static_cast<const bf16_t*>(z)[r * row + h]);
+    return 1.0f / (1.0f + expf(-v));
+  }
+};
 
 // ---- a product per head -------------------------------------------------------------------------------------------
 // out[t, h, n] = sum_k a[t, h, k] * w[h, n, k]: 64 x 64 outputs a workgroup of 256 threads (4 x 4 a thread), k in steps
@@ -103,7 +155,7 @@ constexpr int kHT = 64, kHK = 16;
 template <typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void heads_gemm_kernel(const TA* __restrict__ a, long a_row, long a_head,
                                                          const TW* __restrict__ w, TO* __restrict__ out, long o_row,
-                                                         long o_head, int m, int n, int k) {
+                                                         long o_head, int m, int n, int k, const HeadGate gate) {
   __shared__ float a_s[kHK][kHT + 1], w_s[kHK][kHT + 1];
   const int h = blockIdx.z, m0 = blockIdx.x * kHT, n0 = blockIdx.y * kHT;
   const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
@@ -135,7 +187,7 @@ __global__ __launch_bounds__(256) void heads_gemm_kernel(const TA* __restrict__ 
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int r = m0 + ty * 4 + i, c = n0 + tx * 4 + j;
-      if (r < m && c < n) out[r * o_row + h * o_head + c] = from_float<TO>(acc[i][j]);
+      if (r < m && c < n) out[r * o_row + h * o_head + c] = from_float<TO>(acc[i][j] * gate.of(r, h));
     }
 }
 
@@ -156,7 +208,7 @@ __device__ inline uint4 load_slots(const float* p) {
 template <typename TA, typename TO, int NB, int KW>
 __global__ __launch_bounds__(kWave * KW) void heads_mfma_kernel(const TA* __restrict__ a, long a_row, long a_head,
                                                                 const bf16_t* __restrict__ w, TO* __restrict__ out, long o_row,
-                                                                long o_head, int m, int n, int k) {
+                                                                long o_head, int m, int n, int k, const HeadGate gate) {
   __shared__ floatx4 sums[KW > 1 ? KW : 1][NB][kWave];
   const int h = blockIdx.z, m0 = blockIdx.x * 16, n0 = blockIdx.y * 16 * NB;
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -194,13 +246,16 @@ __global__ __launch_bounds__(kWave * KW) void heads_mfma_kernel(const TA* __rest
       for (int other = 1; other < KW; ++other) acc[nb] += sums[other][nb][lane];
   }
   // a lane holds column c of every block and rows 4g .. 4g + 3
+  float by[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) by[i] = m0 + 4 * g + i < m ? gate.of(m0 + 4 * g + i, h) : 1.0f;
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb) {
     if (!col_there[nb]) continue;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int r = m0 + 4 * g + i;
-      if (r < m) out[r * o_row + h * o_head + n0 + nb * 16 + c] = from_float<TO>(acc[nb][i]);
+      if (r < m) out[r * o_row + h * o_head + n0 + nb * 16 + c] = from_float<TO>(acc[nb][i] * by[i]);
     }
   }
 }
@@ -320,37 +375,45 @@ extern "C" int bc4g_latent_angles(const int32_t* positions, float* table, int n_
 extern "C" int bc4g_latent_prepare(const void* q, const void* dkv, int dtype, const float* g, float eps,
                                    const float* angles, const int32_t* slot_map, void* cache, float* q_lat,
                                    int n_rows, int heads, int plain, int rot, int rank, int dims, long q_row, long dkv_row,
+                                   int halves, const void* low, const float* low_g, void* low_out, int low_rank, long low_row,
                                    void* stream) {
   BC4G_REQUIRE(n_rows >= 0 && heads > 0 && plain >= 0 && rot >= 0 && rank > 0, "latent_prepare: bad sizes T=%d heads=%d "
                "plain=%d rot=%d rank=%d", n_rows, heads, plain, rot, rank);
   BC4G_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= rot && dims <= 8192,
                "latent_prepare: %d rotated dimensions of %d (even, at most the rotated part)", dims, rot);
-  BC4G_REQUIRE((rot == 0 || (q && q_lat)) && (angles || dims == 0) && (!cache || (dkv && g && slot_map)),
+  BC4G_REQUIRE(!low || (low_g && low_out && low_rank > 0 && low_row >= low_rank), "latent_prepare: a query latent of %d numbers, rows %ld apart",
+               low_rank, low_row);
+  BC4G_REQUIRE((rot == 0 || !q == !q_lat) && (angles || dims == 0) && (!cache || (dkv && g && slot_map)),
                "latent_prepare: a tensor is missing");
-  BC4G_REQUIRE((rot == 0 || q_row >= static_cast<long>(heads) * (plain + rot)) && (!cache || dkv_row >= rank + rot),
+  BC4G_REQUIRE((rot == 0 || !q || q_row >= static_cast<long>(heads) * (plain + rot)) && (!cache || dkv_row >= rank + rot),
                "latent_prepare: rows shorter than their parts");
-  const int first = cache ? 0 : 1, parts = (cache ? 1 : 0) + (rot > 0 ? 1 : 0);
+  const int parts = (cache ? 1 : 0) | (rot > 0 && q ? 2 : 0) | (low ? 4 : 0);
+  const int n_parts = (parts & 1) + (parts >> 1 & 1) + (parts >> 2 & 1);
   if (n_rows == 0 || parts == 0) return 0;
+  const LowQuery lq{low, low_g, low_out, low_row, low_rank};
   hipStream_t s = static_cast<hipStream_t>(stream);
   const size_t lds = static_cast<size_t>(dims > 0 ? dims : 2) * sizeof(float);
   if (dtype == kF32)
-    latent_prepare_kernel<float><<<dim3(n_rows, parts), kPrepBlock, lds, s>>>(static_cast<const float*>(q), static_cast<const float*>(dkv), g,
+    latent_prepare_kernel<float><<<dim3(n_rows, n_parts), kPrepBlock, lds, s>>>(static_cast<const float*>(q), static_cast<const float*>(dkv), g,
                                                                  eps, angles, slot_map, static_cast<float*>(cache), q_lat,
-                                                                 heads, plain, rot, rank, dims, q_row, dkv_row, first);
+                                                                 heads, plain, rot, rank, dims, q_row, dkv_row, parts, halves, lq);
   else if (dtype == kBF16)
-    latent_prepare_kernel<bf16_t><<<dim3(n_rows, parts), kPrepBlock, lds, s>>>(static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(dkv),
+    latent_prepare_kernel<bf16_t><<<dim3(n_rows, n_parts), kPrepBlock, lds, s>>>(static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(dkv),
                                                                   g, eps, angles, slot_map, static_cast<bf16_t*>(cache),
-                                                                  q_lat, heads, plain, rot, rank, dims, q_row, dkv_row, first);
+                                                                  q_lat, heads, plain, rot, rank, dims, q_row, dkv_row, parts, halves, lq);
   else return fail("latent_prepare: unknown dtype %d", dtype);
   return check_launch("latent_prepare");
 }
 
 extern "C" int bc4g_heads_gemm(const void* a, int a_dtype, long a_row, long a_head, const void* w, int w_dtype, void* out,
-                               int out_dtype, long o_row, long o_head, int m, int n, int k, int heads, void* stream) {
+                               int out_dtype, long o_row, long o_head, int m, int n, int k, int heads, const void* gate, int gate_dtype,
+                               long gate_row, void* stream) {
   BC4G_REQUIRE(m >= 0 && n > 0 && k > 0 && heads > 0 && heads <= 65535, "heads_gemm: bad sizes m=%d n=%d k=%d heads=%d", m, n, k, heads);
   BC4G_REQUIRE(a && w && out && a_row >= k && o_row >= n && a_head >= 0 && o_head >= 0, "heads_gemm: bad operands or strides");
   BC4G_REQUIRE(ceil_div(n, kHT) <= 65535, "heads_gemm: n=%d is beyond the grid limit", n);
+  BC4G_REQUIRE(!gate || (gate_row >= heads && (gate_dtype == kF32 || gate_dtype == kBF16)), "heads_gemm: gate rows %ld apart for %d heads, or an unknown dtype", gate_row, heads);
   if (m == 0) return 0;
+  const HeadGate hg{gate, gate_row, gate_dtype};
   hipStream_t s = static_cast<hipStream_t>(stream);
   // bfloat16 weights with k in whole pieces of 16 bytes: the matrix cores
   const int a_bytes = a_dtype == kBF16 ? 2 : 4;
@@ -365,10 +428,10 @@ extern "C" int bc4g_heads_gemm(const void* a, int a_dtype, long a_row, long a_he
   do {                                                                                                                         \
     if (nb == 1)                                                                                                               \
       heads_mfma_kernel<TA, TO, 1, 4><<<mgrid, 4 * kWave, 0, s>>>(static_cast<const TA*>(a), a_row, a_head, wp,                \
-                                                                  static_cast<TO*>(out), o_row, o_head, m, n, k);              \
+                                                                  static_cast<TO*>(out), o_row, o_head, m, n, k, hg);          \
     else                                                                                                                       \
       heads_mfma_kernel<TA, TO, 4, 1><<<mgrid, kWave, 0, s>>>(static_cast<const TA*>(a), a_row, a_head, wp,                    \
-                                                              static_cast<TO*>(out), o_row, o_head, m, n, k);                  \
+                                                              static_cast<TO*>(out), o_row, o_head, m, n, k, hg);              \
   } while (0)
     if (a_dtype == kBF16 && out_dtype == kF32) BC4G_HM(bf16_t, float);
     else if (a_dtype == kBF16) BC4G_HM(bf16_t, bf16_t);
@@ -380,7 +443,7 @@ extern "C" int bc4g_heads_gemm(const void* a, int a_dtype, long a_row, long a_he
   dim3 grid(ceil_div(m, kHT), ceil_div(n, kHT), heads);
 #define BC4G_HG(TA, TW, TO)                                                                                              \
   heads_gemm_kernel<TA, TW, TO><<<grid, 256, 0, s>>>(static_cast<const TA*>(a), a_row, a_head, static_cast<const TW*>(w), \
-                                                     static_cast<TO*>(out), o_row, o_head, m, n, k)
+                                                     static_cast<TO*>(out), o_row, o_head, m, n, k, hg)
   const int code = a_dtype * 4 + w_dtype * 2 + out_dtype;
   BC4G_REQUIRE(a_dtype >= 0 && a_dtype <= 1 && w_dtype >= 0 && w_dtype <= 1 && out_dtype >= 0 && out_dtype <= 1,
                "heads_gemm: unknown dtypes %d, %d, %d", a_dtype, w_dtype, out_dtype);

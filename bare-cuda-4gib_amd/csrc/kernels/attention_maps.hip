@@ -64,7 +64,7 @@ __global__ __launch_bounds__(kNW * kWave) void attention_maps_kernel(
     const float* __restrict__ q, long q_row, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
     const int32_t* __restrict__ block_table, int table_stride, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ positions, float lambda, int normalize, float eps, float factor,
-    const void* __restrict__ gate, int gate_dtype, long gate_row, int gate_act, void* __restrict__ out, int out_dtype,
+    const void* __restrict__ gate, int gate_dtype, long gate_row, int gate_act, void* __restrict__ out, int out_dtype, long out_row,
     int n_heads, int n_kv_heads, int dim, int vdim, int page_tokens, int window, int keep_first, float scale,
     const float* __restrict__ sink, const float* __restrict__ far1, const float* __restrict__ far2, int block, float cap,
     const float* __restrict__ point) {
@@ -275,7 +275,7 @@ __global__ __launch_bounds__(kNW * kWave) void attention_maps_kernel(
     if (c >= vdim || !writer) continue;
     float r = o[i] * mult;
     if (gate) r *= gate_of(gate, gate_dtype, row * gate_row + static_cast<long>(head) * vdim + c, gate_act);
-    const long at = (static_cast<long>(row) * n_heads + head) * vdim + c;
+    const long at = row * out_row + static_cast<long>(head) * vdim + c;
     if (out_dtype == kF32) static_cast<float*>(out)[at] = r;
     else static_cast<bf16_t*>(out)[at] = from_float<bf16_t>(r);
   }
@@ -290,7 +290,7 @@ extern "C" int bc4g_attention_maps(const float* q, long q_row, const void* k_cac
                                    const int32_t* block_table, int table_stride, const int32_t* row_seq,
                                    const int32_t* positions, float lambda, int normalize, float eps, float factor,
                                    const void* gate, int gate_dtype, long gate_row, int gate_act, void* out, int out_dtype,
-                                   int n_rows, int n_heads, int n_kv_heads, int maps, int dim, int vdim, int page_tokens,
+                                   long out_row, int n_rows, int n_heads, int n_kv_heads, int maps, int dim, int vdim, int page_tokens,
                                    int window, int keep_first, float scale, int waves, const float* sink,
                                    const float* far1, const float* far2, int block, float cap, const float* point,
                                    void* stream) {
@@ -304,7 +304,7 @@ extern "C" int bc4g_attention_maps(const float* q, long q_row, const void* k_cac
                table_stride, window, keep_first);
   BC4G_REQUIRE(q && k_cache && v_cache && block_table && row_seq && positions && out &&
                q_row >= static_cast<long>(n_heads) * maps * dim && (!gate || gate_row >= static_cast<long>(n_heads) * vdim) &&
-               (gate_act == 1 || gate_act == 2 || !gate) && (out_dtype == kF32 || out_dtype == kBF16) &&
+               out_row >= static_cast<long>(n_heads) * vdim && (gate_act == 1 || gate_act == 2 || !gate) && (out_dtype == kF32 || out_dtype == kBF16) &&
                (!gate || gate_dtype == kF32 || gate_dtype == kBF16),
                "attention_maps: a tensor is missing, a row is shorter than its heads, or a dtype is unknown");
   BC4G_REQUIRE((far1 == nullptr) == (far2 == nullptr), "attention_maps: the distance penalty needs both of its vectors");
@@ -324,7 +324,7 @@ extern "C" int bc4g_attention_maps(const float* q, long q_row, const void* k_cac
 #define BC4G_MAPS_E(T, M, W, V, E)                                                                                        \
   attention_maps_kernel<T, M, W, V, E><<<grid, waves * kWave, 0, s>>>(q, q_row, static_cast<const T*>(k_cache), static_cast<const T*>(v_cache), \
                                                      block_table, table_stride, row_seq, positions, lambda, normalize, eps, \
-                                                     factor, gate, gate_dtype, gate_row, gate_act, out, out_dtype, n_heads,  \
+                                                     factor, gate, gate_dtype, gate_row, gate_act, out, out_dtype, out_row, n_heads,  \
                                                      n_kv_heads, dim, vdim, page_tokens, window, keep_first, scale, sink, far1, far2, block, cap, point)
   if (cache_dtype == kF32) {
     if (maps == 1) BC4G_MAPS(float, 1); else BC4G_MAPS(float, 2);

@@ -7,7 +7,7 @@
 //             i + half), the frequencies given by the caller (so any scaling of them is the caller's), both multiplied
 //             by an amplitude; angles in double.
 //   prepare   per (row, head): + bias, RMS norm over the head with a weight, rotation (either pairing), division by the
-//             root mean square after the rotation, a factor -- each optional -- into a dense tensor or into the pages
+//             root mean square after the rotation, a factor, one that grows with the position -- each optional -- into a dense tensor or into the pages
 //             of a cache.
 //   finish    per (row, head): o / rms(o) (* weight) * factor * act(gate).
 //
@@ -140,7 +140,12 @@ __global__ __launch_bounds__(kWave) void heads_prepare_kernel(const PrepareSecti
     ss_after = fmaf(v, v, ss_after);
   }
   // (unit_after: the head divided by its root mean square as it stands after the rotation, no weight)
-  const float last = p.unit_after ? p.factor / sqrtf(wave_sum(ss_after) / static_cast<float>(dim) + p.eps) : p.factor;
+  float last = p.unit_after ? p.factor / sqrtf(wave_sum(ss_after) / static_cast<float>(dim) + p.eps) : p.factor;
+  // (the temperature of a position: 1 + coef ln(floor((pos + 1) / every) + 1), the quotient in double so that the floor is the number's own)
+  if (p.positions) {
+    const double steps = floor((static_cast<double>(p.positions[row]) + 1.0) / p.temp_every);
+    last *= 1.0f + p.temp_coef * logf(static_cast<float>(steps) + 1.0f);
+  }
 #pragma unroll
   for (int n = 0; n < kMaxHead / kWave; ++n) {
     const int c = lane + n * kWave;
@@ -387,6 +392,7 @@ extern "C" int bc4g_heads_prepare_many(const bc4g_prepare_section* sections, int
                  (p.slot_map ? p.page_tokens > 0 : p.out_row >= static_cast<long>(p.heads) * p.dim) &&
                  (p.in_dtype == kF32 || p.in_dtype == kBF16) && (p.out_dtype == kF32 || p.out_dtype == kBF16),
                  "heads_prepare: a tensor is missing, a row is shorter than its heads, or a dtype is unknown");
+    BC4G_REQUIRE(!p.positions || p.temp_every > 0.0, "heads_prepare: a temperature needs a positive number of positions, got %g", p.temp_every);
     all.s[i] = p;
     heads += p.heads;
   }
@@ -403,7 +409,7 @@ extern "C" int bc4g_heads_prepare(const void* in, int in_dtype, long in_row, con
                                   const int32_t* slot_map, int page_tokens, long page_stride, long head_stride,
                                   long token_stride, int n_rows, int heads, int dim, void* stream) {
   const bc4g_prepare_section one{in, bias, norm_w, table, out, slot_map, in_row, out_row, page_stride, head_stride, token_stride,
-                                 in_dtype, out_dtype, half, page_tokens, heads, dim, eps, factor, 0, 0, 0};
+                                 in_dtype, out_dtype, half, page_tokens, heads, dim, eps, factor, 0, 0, 0, 0.f, 0.0, nullptr};
   return bc4g_heads_prepare_many(&one, 1, n_rows, stream);
 }
 

@@ -126,6 +126,7 @@ __global__ __launch_bounds__(256) void rmsnorm_rows_kernel(const float* __restri
 // workgroups (bc4g_gemm_mfma_parts).
 template <typename TW, typename TO, int CHUNKS>
 __global__ __launch_bounds__(256) void rmsnorm_sum_rows_kernel(float* __restrict__ x, const float* __restrict__ parts, int n_parts,
+                                                               const float* __restrict__ bias,
                                                                const TW* __restrict__ w, TO* __restrict__ out, int n_rows,
                                                                int hidden, float eps) {
   __shared__ float scratch[16];
@@ -139,6 +140,11 @@ __global__ __launch_bounds__(256) void rmsnorm_sum_rows_kernel(float* __restrict
     const int i = (c * 256 + threadIdx.x) * 8;
     if (i < hidden) {
       float4 a = *reinterpret_cast<const float4*>(xr + i), b = *reinterpret_cast<const float4*>(xr + i + 4);
+      if (bias != nullptr) {
+        const float4 ba = *reinterpret_cast<const float4*>(bias + i), bb = *reinterpret_cast<const float4*>(bias + i + 4);
+        a.x += ba.x; a.y += ba.y; a.z += ba.z; a.w += ba.w;
+        b.x += bb.x; b.y += bb.y; b.z += bb.z; b.w += bb.w;
+      }
       for (int p = 0; p < n_parts; ++p) {
         const float* pr = parts + p * part_stride + at + i;
         const float4 pa = *reinterpret_cast<const float4*>(pr), pb = *reinterpret_cast<const float4*>(pr + 4);
@@ -184,7 +190,7 @@ __global__ __launch_bounds__(256) void rmsnorm_sum_rows_kernel(float* __restrict
 // weight-streaming kernel produces and consumes).
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, long total, int inter,
-                              int interleaved) {
+                              int interleaved, int act) {
   const long stride = static_cast<long>(blockDim.x) * gridDim.x;
   for (long idx = blockIdx.x * static_cast<long>(blockDim.x) + threadIdx.x; idx < total; idx += stride) {
     const long t = idx / inter;
@@ -193,7 +199,9 @@ __global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, lon
     const long ui = interleaved ? gi + 8 : inter + i;
     const float g = to_float(gu[t * 2 * inter + gi]);
     const float u = to_float(gu[t * 2 * inter + ui]);
-    out[idx] = from_float<T>((g / (1.0f + expf(-g))) * u);
+    // act 0: the silu, 1: the gelu written with tanh
+    const float a = act == 1 ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g));
+    out[idx] = from_float<T>(a * u);
   }
 }
 
@@ -722,10 +730,11 @@ extern "C" int bc4g_rmsnorm_groups(const float* x, const int32_t* rows, const vo
   return check_launch("rmsnorm");
 }
 
-extern "C" int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const void* w, int w_dtype, void* out,
+extern "C" int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const float* bias, const void* w, int w_dtype, void* out,
                                 int out_dtype, int n_rows, int hidden, float eps, void* stream) {
   BC4G_REQUIRE(n_rows >= 0 && hidden > 0 && hidden % 8 == 0 && hidden <= 8192 && n_parts >= 1 && n_parts <= 16,
                "rmsnorm_sum: rows=%d of H=%d (a multiple of 8, at most 8192) in %d parts (1 to 16)", n_rows, hidden, n_parts);
+  BC4G_REQUIRE(!bias || reinterpret_cast<uintptr_t>(bias) % 16 == 0, "rmsnorm_sum: the bias must lie on a 16-byte boundary");
   if (n_rows == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int chunks = (hidden + 2047) / 2048;
@@ -733,9 +742,9 @@ extern "C" int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const
   do {                                                                                                                    \
     const TW* wp = static_cast<const TW*>(w);                                                                             \
     TO* op = static_cast<TO*>(out);                                                                                       \
-    if (chunks == 1) rmsnorm_sum_rows_kernel<TW, TO, 1><<<n_rows, 256, 0, s>>>(x, parts, n_parts, wp, op, n_rows, hidden, eps);      \
-    else if (chunks == 2) rmsnorm_sum_rows_kernel<TW, TO, 2><<<n_rows, 256, 0, s>>>(x, parts, n_parts, wp, op, n_rows, hidden, eps); \
-    else rmsnorm_sum_rows_kernel<TW, TO, 4><<<n_rows, 256, 0, s>>>(x, parts, n_parts, wp, op, n_rows, hidden, eps);                  \
+    if (chunks == 1) rmsnorm_sum_rows_kernel<TW, TO, 1><<<n_rows, 256, 0, s>>>(x, parts, n_parts, bias, wp, op, n_rows, hidden, eps);      \
+    else if (chunks == 2) rmsnorm_sum_rows_kernel<TW, TO, 2><<<n_rows, 256, 0, s>>>(x, parts, n_parts, bias, wp, op, n_rows, hidden, eps); \
+    else rmsnorm_sum_rows_kernel<TW, TO, 4><<<n_rows, 256, 0, s>>>(x, parts, n_parts, bias, wp, op, n_rows, hidden, eps);                  \
   } while (0)
   if (w_dtype == kF32 && out_dtype == kBF16) BC4G_RMS_SUM(float, bf16_t);
   else if (w_dtype == kBF16 && out_dtype == kBF16) BC4G_RMS_SUM(bf16_t, bf16_t);
@@ -744,8 +753,9 @@ extern "C" int bc4g_rmsnorm_sum(float* x, const float* parts, int n_parts, const
   return check_launch("rmsnorm_sum");
 }
 
-extern "C" int bc4g_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int interleaved,
+extern "C" int bc4g_swiglu(const void* gu, void* out, int dtype, int n_tokens, int inter, int interleaved, int act,
                            void* stream) {
+  BC4G_REQUIRE(act == 0 || act == 1, "swiglu: activation %d (0: silu, 1: gelu with tanh)", act);
   BC4G_REQUIRE(n_tokens >= 0 && inter > 0, "swiglu: bad sizes T=%d I=%d", n_tokens, inter);
   BC4G_REQUIRE(!interleaved || inter % 8 == 0, "swiglu: the interleaved layout needs I=%d to be a multiple of 8", inter);
   if (n_tokens == 0) return 0;
@@ -753,10 +763,10 @@ extern "C" int bc4g_swiglu(const void* gu, void* out, int dtype, int n_tokens, i
   const long total = static_cast<long>(n_tokens) * inter;
   if (dtype == kF32) {
     swiglu_kernel<float><<<grid_for(total), kBlock, 0, s>>>(static_cast<const float*>(gu),
-                                                            static_cast<float*>(out), total, inter, interleaved);
+                                                            static_cast<float*>(out), total, inter, interleaved, act);
   } else if (dtype == kBF16) {
     swiglu_kernel<bf16_t><<<grid_for(total), kBlock, 0, s>>>(static_cast<const bf16_t*>(gu),
-                                                             static_cast<bf16_t*>(out), total, inter, interleaved);
+                                                             static_cast<bf16_t*>(out), total, inter, interleaved, act);
   } else {
     return fail("swiglu: unknown dtype %d", dtype);
   }

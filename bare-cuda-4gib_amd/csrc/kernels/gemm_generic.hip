@@ -19,7 +19,7 @@ constexpr int kFewRows = 16;   // rows up to which the small tile serves
 template <typename TA, typename TW, typename TO, bool kAccumulate, int kPerThread, int kStepK>
 __global__ __launch_bounds__(256) void gemm_generic_kernel(const TA* __restrict__ a,
                                                            const TW* __restrict__ w,
-                                                           TO* __restrict__ out, int m, int n, int k) {
+                                                           TO* __restrict__ out, const float* __restrict__ bias, int m, int n, int k) {
   constexpr int kTile = 16 * kPerThread;   // output tile per block, both ways
   // k-major tiles, padded so that the 16 threads of a row group hit different banks.
   __shared__ float as[kStepK][kTile + 1];
@@ -85,7 +85,7 @@ __global__ __launch_bounds__(256) void gemm_generic_kernel(const TA* __restrict_
       const long gn = n0 + tx * kPerThread + j;
       if (gn >= n) continue;
       if constexpr (kAccumulate) {
-        out[gm * n + gn] = from_float<TO>(to_float(out[gm * n + gn]) + acc[i][j]);
+        out[gm * n + gn] = from_float<TO>(to_float(out[gm * n + gn]) + (bias != nullptr ? bias[gn] : 0.f) + acc[i][j]);
       } else {
         out[gm * n + gn] = from_float<TO>(acc[i][j]);
       }
@@ -94,14 +94,14 @@ __global__ __launch_bounds__(256) void gemm_generic_kernel(const TA* __restrict_
 }
 
 template <typename TA, typename TW, typename TO, bool kAcc>
-void launch(const void* a, const void* w, void* out, int m, int n, int k, hipStream_t s) {
+void launch(const void* a, const void* w, void* out, const float* bias, int m, int n, int k, hipStream_t s) {
   if (m <= kFewRows) {
     gemm_generic_kernel<TA, TW, TO, kAcc, 1, 64><<<dim3(ceil_div(n, 16), 1), 256, 0, s>>>(
-        static_cast<const TA*>(a), static_cast<const TW*>(w), static_cast<TO*>(out), m, n, k);
+        static_cast<const TA*>(a), static_cast<const TW*>(w), static_cast<TO*>(out), bias, m, n, k);
     return;
   }
   gemm_generic_kernel<TA, TW, TO, kAcc, 4, 16><<<dim3(ceil_div(n, 64), ceil_div(m, 64)), 256, 0, s>>>(
-      static_cast<const TA*>(a), static_cast<const TW*>(w), static_cast<TO*>(out), m, n, k);
+      static_cast<const TA*>(a), static_cast<const TW*>(w), static_cast<TO*>(out), bias, m, n, k);
 }
 
 }  // namespace
@@ -110,31 +110,32 @@ void launch(const void* a, const void* w, void* out, int m, int n, int k, hipStr
 using namespace bc4g;
 
 extern "C" int bc4g_gemm_generic(const void* a, int a_dtype, const void* w, int w_dtype, void* out,
-                                 int out_dtype, int accumulate, int m, int n, int k, void* stream) {
+                                 int out_dtype, int accumulate, const float* bias, int m, int n, int k, void* stream) {
   BC4G_REQUIRE(m >= 0 && n > 0 && k > 0, "gemm: bad sizes M=%d N=%d K=%d", m, n, k);
   BC4G_REQUIRE(!accumulate || out_dtype == kF32, "gemm: accumulation needs a float32 output");
+  BC4G_REQUIRE(!bias || accumulate, "gemm: only an adding product takes a bias");
   BC4G_REQUIRE(ceil_div(m, 64) <= 65535, "gemm: M=%d is beyond the grid limit", m);
   if (m == 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int key = a_dtype * 100 + w_dtype * 10 + out_dtype;
   switch (key) {
     case 0:   // f32 x f32 -> f32
-      if (accumulate) launch<float, float, float, true>(a, w, out, m, n, k, s);
-      else launch<float, float, float, false>(a, w, out, m, n, k, s);
+      if (accumulate) launch<float, float, float, true>(a, w, out, bias, m, n, k, s);
+      else launch<float, float, float, false>(a, w, out, bias, m, n, k, s);
       break;
     case 110:  // bf16 x bf16 -> f32
-      if (accumulate) launch<bf16_t, bf16_t, float, true>(a, w, out, m, n, k, s);
-      else launch<bf16_t, bf16_t, float, false>(a, w, out, m, n, k, s);
+      if (accumulate) launch<bf16_t, bf16_t, float, true>(a, w, out, bias, m, n, k, s);
+      else launch<bf16_t, bf16_t, float, false>(a, w, out, bias, m, n, k, s);
       break;
     case 111:  // bf16 x bf16 -> bf16
-      launch<bf16_t, bf16_t, bf16_t, false>(a, w, out, m, n, k, s);
+      launch<bf16_t, bf16_t, bf16_t, false>(a, w, out, bias, m, n, k, s);
       break;
     case 100:  // bf16 x f32 -> f32
-      if (accumulate) launch<bf16_t, float, float, true>(a, w, out, m, n, k, s);
-      else launch<bf16_t, float, float, false>(a, w, out, m, n, k, s);
+      if (accumulate) launch<bf16_t, float, float, true>(a, w, out, bias, m, n, k, s);
+      else launch<bf16_t, float, float, false>(a, w, out, bias, m, n, k, s);
       break;
     case 101:  // bf16 x f32 -> bf16
-      launch<bf16_t, float, bf16_t, false>(a, w, out, m, n, k, s);
+      launch<bf16_t, float, bf16_t, false>(a, w, out, bias, m, n, k, s);
       break;
     default:
       return fail("gemm: unsupported dtypes a=%d w=%d out=%d", a_dtype, w_dtype, out_dtype);

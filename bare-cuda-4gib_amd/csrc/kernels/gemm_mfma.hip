@@ -43,9 +43,16 @@ constexpr int kXcds = 8;
 // product that last added to the residual left it, with every row's sum of squares in parts): a row's sums are
 // multiplied by 1 / sqrt(sum of squares / k + eps) before the activation (operands straight into LDS only).
 // kSquaredReluBf16: out = max(sum, 0)^2, stored as bfloat16.
+// kGegluBf16, kGegluScaledBf16: as the two SwiGLU epilogues, with the gelu written with tanh for the silu.
+// kAccumF32 may add a number a column beside the product (bias).
 enum Epilogue : int {
-  kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSwigluScaledBf16 = 5, kSquaredReluBf16 = 6
+  kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSwigluScaledBf16 = 5, kSquaredReluBf16 = 6,
+  kGegluBf16 = 7, kGegluScaledBf16 = 8
 };
+constexpr bool gated(int epi) { return epi == kSwigluBf16 || epi == kSwigluScaledBf16 || epi == kGegluBf16 || epi == kGegluScaledBf16; }
+constexpr bool row_scaled(int epi) { return epi == kSwigluScaledBf16 || epi == kGegluScaledBf16; }
+template <int EPI>
+__device__ inline float gate_act(float z) { return EPI == kGegluBf16 || EPI == kGegluScaledBf16 ? gelu_tanh_quick(z) : silu_quick(z); }
 
 __device__ inline float squared_relu(float v) {
   const float z = fmaxf(v, 0.f);
@@ -58,6 +65,7 @@ struct RowScaleArgs {
   const float* parts;         // [blocks][stride]: block b's share of every row's sum of squares
   int blocks, stride;
   float eps;
+  const float* bias;          // kAccumF32: [n], joins every row's sums (null: none)
 };
 // a patch's rows' sums in LDS ([kPartSums][stride], from the patch's first row on) and what finishes them
 struct RowScale {
@@ -96,9 +104,9 @@ __device__ inline void tile_of(int block, int m_blocks, int n_blocks, int& bm, i
 // Stores ROWS x COLS floats (stride COLS + 4) from LDS with the epilogue, THREADS threads together.
 template <int EPI, int THREADS, int ROWS, int COLS>
 __device__ inline void store_patch(const float* patch, void* __restrict__ out, int m, int n, long m0, long n0, int tid,
-                                   const RowScale& rs = RowScale{}) {
+                                   const RowScale& rs = RowScale{}, const float* bias = nullptr) {
   constexpr int kStride = COLS + 4;
-  if constexpr (EPI == kSwigluBf16 || EPI == kSwigluScaledBf16) {
+  if constexpr (gated(EPI)) {
     // (a block of 16 columns -- eight gates, then their eight ups -- a thread: eight outputs, stored at once)
     const long n_out = n / 2;
     for (int c = tid; c < ROWS * (COLS / 16); c += THREADS) {
@@ -109,7 +117,7 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
       const floatx4 g0 = *reinterpret_cast<const floatx4*>(src), g1 = *reinterpret_cast<const floatx4*>(src + 4);
       const floatx4 u0 = *reinterpret_cast<const floatx4*>(src + 8), u1 = *reinterpret_cast<const floatx4*>(src + 12);
       float scale = 1.f;
-      if constexpr (EPI == kSwigluScaledBf16) {
+      if constexpr (row_scaled(EPI)) {
         float ssq = 0.f;
 #pragma unroll
         for (int j = 0; j < kPartSums; ++j) ssq += rs.sums[j * rs.stride + row];
@@ -118,8 +126,8 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
       float v[8];
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        v[e] = silu_quick(g0[e] * scale) * (u0[e] * scale);
-        v[4 + e] = silu_quick(g1[e] * scale) * (u1[e] * scale);
+        v[e] = gate_act<EPI>(g0[e] * scale) * (u0[e] * scale);
+        v[4 + e] = gate_act<EPI>(g1[e] * scale) * (u1[e] * scale);
       }
       bf16_t* dst = static_cast<bf16_t*>(out) + gm * n_out + (gn / 16) * 8;
       if (n_out % 8 == 0) {
@@ -163,6 +171,12 @@ __device__ inline void store_patch(const float* patch, void* __restrict__ out, i
       if constexpr (EPI == kSquaredReluBf16) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = squared_relu(v[e]);
+      }
+      if constexpr (EPI == kAccumF32) {
+        if (bias != nullptr) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] += gn + e < n ? bias[gn + e] : 0.f;
+        }
       }
       const long o = gm * n + gn;
       if (vec) {
@@ -304,7 +318,7 @@ struct StagedTile {
 template <int EPI>
 __global__ __launch_bounds__(256, 2) void gemm_mfma_staged_kernel(
     const bf16_t* __restrict__ a, const bf16_t* __restrict__ w, void* __restrict__ out, int m, int n, int k,
-    int m_blocks, int n_blocks) {
+    int m_blocks, int n_blocks, const float* __restrict__ bias) {
   constexpr int SETS = 2, kRows = kBM, kThreads = 256;   // SETS register sets: SETS - 1 k-steps in flight while one is written
   constexpr int kChunkRows = kThreads / 8;           // rows one chunk of a thread's loads covers
   constexpr int kChunksA = kRows / kChunkRows, kChunksW = kBN / kChunkRows;
@@ -435,7 +449,7 @@ __global__ __launch_bounds__(256, 2) void gemm_mfma_staged_kernel(
         tile_out[(wm * 64 + i * 32 + 8 * (r / 4) + 4 * (lane / 32) + r % 4) * kOutStride + wn * 64 + j * 32 + lane % 32] =
             acc[i][j][r];
   lds_barrier();
-  store_patch<EPI, kThreads, kBM, kBN>(tile_out, out, m, n, m0, n0, tid);
+  store_patch<EPI, kThreads, kBM, kBN>(tile_out, out, m, n, m0, n0, tid, RowScale{}, bias);
 }
 
 // ---- operands straight into LDS ---------------------------------------------------------------
@@ -575,8 +589,8 @@ __global__ __launch_bounds__(64 * WM * WN, MINWG) void gemm_mfma_direct_kernel(
   // together), beside the first operands' way into LDS.  (The compiler's wait for these loads knows nothing of the
   // operands asked for before them and so waits for those too: loads return in the order asked.  By the loop's own
   // waits, which count the operands' loads alone, these are done.)
-  __shared__ __align__(16) float part_sum[EPI == kSwigluScaledBf16 ? kPartSums * RA : 4];
-  if constexpr (EPI == kSwigluScaledBf16) {
+  __shared__ __align__(16) float part_sum[row_scaled(EPI) ? kPartSums * RA : 4];
+  if constexpr (row_scaled(EPI)) {
     static_assert(kPartSums * RA % S::kThreads == 0 && kPartSums * RA / 4 <= S::kThreads, "whole chains a thread");
     constexpr int kAhead = 16;              // parts of a chain asked for together: one way to memory and back for 128 parts
     // Four rows a thread where the parts' rows allow loads of 16 bytes (a tile begins at a multiple of 64 rows): a CU
@@ -686,11 +700,11 @@ __global__ __launch_bounds__(64 * WM * WN, MINWG) void gemm_mfma_direct_kernel(
       for (int r = 0; r < 16; ++r) patch[(8 * (r / 4) + 4 * (lane / 32) + r % 4) * kStride + j * 32 + lane % 32] = acc[i][j][r];
     if constexpr (EPI == kRopeKvBf16)
       store_patch_rope<kWave, 32, 32 * TN>(patch, static_cast<bf16_t*>(out), m, n, m0 + (wm * TM + i) * 32, n0 + wn * TN * 32, lane, ra);
-    else if constexpr (EPI == kSwigluScaledBf16)
+    else if constexpr (row_scaled(EPI))
       store_patch<EPI, kWave, 32, 32 * TN>(patch, out, m, n, m0 + (wm * TM + i) * 32, n0 + wn * TN * 32, lane,
                                            RowScale{part_sum + (wm * TM + i) * 32, RA, 1.0f / static_cast<float>(k), rows.eps});
     else
-      store_patch<EPI, kWave, 32, 32 * TN>(patch, out, m, n, m0 + (wm * TM + i) * 32, n0 + wn * TN * 32, lane);
+      store_patch<EPI, kWave, 32, 32 * TN>(patch, out, m, n, m0 + (wm * TM + i) * 32, n0 + wn * TN * 32, lane, RowScale{}, rows.bias);
   }
 }
 
@@ -774,15 +788,15 @@ bool direct_operands(const void* ap, const void* wp, int k) {
 // whole steps of 64, operands on 16-byte boundaries); else the weight by rows, for the kernel that stages its tiles
 // through registers (any k that is a multiple of 8).
 template <int EPI>
-int launch_tiled(const bf16_t* ap, const bf16_t* wp, void* out, int m, int n, int k, hipStream_t s, int w_packed) {
+int launch_tiled(const bf16_t* ap, const bf16_t* wp, void* out, const float* bias, int m, int n, int k, hipStream_t s, int w_packed) {
   if (w_packed) {
     if (!direct_operands(ap, wp, k))
       return fail("gemm_mfma: a packed weight needs k in whole steps of 64 and operands on 16-byte boundaries (K=%d)", k);
-    return launch_direct_form<EPI>(ap, wp, out, m, n, k, s);
+    return launch_direct_form<EPI>(ap, wp, out, m, n, k, s, RopeKvArgs{}, RowScaleArgs{nullptr, 0, 0, 0.f, bias});
   }
   const long m_blocks = (m + kBM - 1) / kBM, n_blocks = (n + kBN - 1) / kBN;
   gemm_mfma_staged_kernel<EPI><<<dim3(static_cast<unsigned>(m_blocks * n_blocks)), dim3(256), 0, s>>>(
-      ap, wp, out, m, n, k, static_cast<int>(m_blocks), static_cast<int>(n_blocks));
+      ap, wp, out, m, n, k, static_cast<int>(m_blocks), static_cast<int>(n_blocks), bias);
   return 0;
 }
 
@@ -791,10 +805,11 @@ int launch_tiled(const bf16_t* ap, const bf16_t* wp, void* out, int m, int n, in
 
 using namespace bc4g;
 
-extern "C" int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* out, int epilogue, int m, int n, int k,
+extern "C" int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* out, const float* bias, int epilogue, int m, int n, int k,
                               void* stream) {
   BC4G_REQUIRE(m >= 0 && n > 0 && k > 0 && k % 8 == 0, "gemm_mfma: K=%d must be a positive multiple of 8 (M=%d N=%d)",
                k, m, n);
+  BC4G_REQUIRE(!bias || epilogue == kAccumF32, "gemm_mfma: only the adding epilogue takes a bias");
   if (m == 0) return 0;
   BC4G_REQUIRE(((m + 63L) / 64) * ((n + 63L) / 64) <= 2147483647L, "gemm_mfma: too many tiles");
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -802,13 +817,15 @@ extern "C" int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* 
   const bf16_t* wp = static_cast<const bf16_t*>(w);
   int e = 0;
   switch (epilogue) {
-    case kStoreBf16: e = launch_tiled<kStoreBf16>(ap, wp, out, m, n, k, s, w_packed); break;
-    case kStoreF32: e = launch_tiled<kStoreF32>(ap, wp, out, m, n, k, s, w_packed); break;
-    case kAccumF32: e = launch_tiled<kAccumF32>(ap, wp, out, m, n, k, s, w_packed); break;
-    case kSquaredReluBf16: e = launch_tiled<kSquaredReluBf16>(ap, wp, out, m, n, k, s, w_packed); break;
+    case kStoreBf16: e = launch_tiled<kStoreBf16>(ap, wp, out, bias, m, n, k, s, w_packed); break;
+    case kStoreF32: e = launch_tiled<kStoreF32>(ap, wp, out, bias, m, n, k, s, w_packed); break;
+    case kAccumF32: e = launch_tiled<kAccumF32>(ap, wp, out, bias, m, n, k, s, w_packed); break;
+    case kSquaredReluBf16: e = launch_tiled<kSquaredReluBf16>(ap, wp, out, bias, m, n, k, s, w_packed); break;
     case kSwigluBf16:
-      BC4G_REQUIRE(n % 16 == 0, "gemm_mfma: SwiGLU needs blocks of eight gate and eight up rows, N=%d is no multiple of 16", n);
-      e = launch_tiled<kSwigluBf16>(ap, wp, out, m, n, k, s, w_packed);
+    case kGegluBf16:
+      BC4G_REQUIRE(n % 16 == 0, "gemm_mfma: a gated product needs blocks of eight gate and eight up rows, N=%d is no multiple of 16", n);
+      if (epilogue == kSwigluBf16) e = launch_tiled<kSwigluBf16>(ap, wp, out, bias, m, n, k, s, w_packed);
+      else e = launch_tiled<kGegluBf16>(ap, wp, out, bias, m, n, k, s, w_packed);
       break;
     default: return fail("gemm_mfma: unknown epilogue %d", epilogue);
   }
@@ -817,16 +834,19 @@ extern "C" int bc4g_gemm_mfma(const void* a, const void* w, int w_packed, void* 
 }
 
 extern "C" int bc4g_gemm_mfma_swiglu_scaled(const void* a, const float* ssq_parts, int ssq_blocks, int ssq_stride, float eps,
-                                            const void* w, int w_packed, void* out, int m, int n, int k, void* stream) {
+                                            const void* w, int w_packed, void* out, int gelu, int m, int n, int k, void* stream) {
   BC4G_REQUIRE(m >= 0 && n > 0 && n % 16 == 0 && k > 0 && direct_operands(a, w, k) && w_packed,
                "gemm_mfma_swiglu_scaled: K=%d must be a multiple of 64, N=%d one of 16, the weight packed and the operands on 16-byte boundaries (M=%d)", k, n, m);
   BC4G_REQUIRE(ssq_parts != nullptr && ssq_blocks > 0 && ssq_stride >= m && eps >= 0.f,
                "gemm_mfma_swiglu_scaled: the sums of squares need %d parts of at least %d rows, and eps must not be negative", ssq_blocks, m);
   if (m == 0) return 0;
   BC4G_REQUIRE(((m + 63L) / 64) * ((n + 63L) / 64) <= 2147483647L, "gemm_mfma_swiglu_scaled: too many tiles");
-  if (int e = launch_direct_form<kSwigluScaledBf16>(static_cast<const bf16_t*>(a), static_cast<const bf16_t*>(w), out, m, n, k,
-                                                     static_cast<hipStream_t>(stream), RopeKvArgs{},
-                                                     RowScaleArgs{ssq_parts, ssq_blocks, ssq_stride, eps}))
+  const bf16_t* ap = static_cast<const bf16_t*>(a);
+  const bf16_t* wp = static_cast<const bf16_t*>(w);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const RowScaleArgs rows{ssq_parts, ssq_blocks, ssq_stride, eps, nullptr};
+  if (int e = gelu ? launch_direct_form<kGegluScaledBf16>(ap, wp, out, m, n, k, s, RopeKvArgs{}, rows)
+                   : launch_direct_form<kSwigluScaledBf16>(ap, wp, out, m, n, k, s, RopeKvArgs{}, rows))
     return e;
   return check_launch("gemm_mfma_swiglu_scaled");
 }

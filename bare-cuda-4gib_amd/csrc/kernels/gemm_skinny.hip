@@ -51,7 +51,9 @@ constexpr int kThreads = kWaves * kWave;
 constexpr int kRedPad = 17;
 constexpr int kStagePad = 8;     // bf16 elements appended to each staged row of x
 
-enum Epilogue : int { kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSquaredReluBf16 = 6 };
+enum Epilogue : int { kStoreBf16 = 0, kStoreF32 = 1, kAccumF32 = 2, kSwigluBf16 = 3, kRopeKvBf16 = 4, kSquaredReluBf16 = 6, kGegluBf16 = 7 };
+// products whose weight holds blocks of eight gate rows and the eight up rows of the same outputs
+constexpr bool gated(int epi) { return epi == kSwigluBf16 || epi == kGegluBf16; }
 
 struct RopeKvArgs {
   const int32_t* positions;   // [m]
@@ -77,6 +79,8 @@ struct SkinnyArgs {
   // prenormed x (plain mode): parts [ssq_blocks][ssq_stride] of the rows' sums of squares (null: x as it is)
   const float* ssq_parts;
   int ssq_blocks, ssq_stride;
+  // kAccumF32: a number a column that joins every row's sums (null: none)
+  const float* bias;
   // kAccumF32: what the RMSNorm after this product needs (emit_g null: nothing)
   const void* emit_g;       // [n] its scale, bfloat16 or float (emit_g_f32)
   bf16_t* emit_x;           // [m, n] bfloat16(new residual * g)
@@ -102,7 +106,7 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
     a.m = min(args.rows_per_block, args.m - static_cast<int>(row0));
     a.x = static_cast<const bf16_t*>(args.x) + row0 * args.k;
     if constexpr (EPI == kStoreBf16 || EPI == kSquaredReluBf16) a.out = static_cast<bf16_t*>(args.out) + row0 * args.n;
-    else if constexpr (EPI == kSwigluBf16) a.out = static_cast<bf16_t*>(args.out) + row0 * (args.n / 2);
+    else if constexpr (gated(EPI)) a.out = static_cast<bf16_t*>(args.out) + row0 * (args.n / 2);
     else if constexpr (EPI == kRopeKvBf16) {
       a.out = static_cast<bf16_t*>(args.out) + row0 * args.rope.n_heads * args.rope.head_dim;
       a.rope.positions = args.rope.positions ? args.rope.positions + row0 : nullptr;
@@ -173,7 +177,9 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
     for (int j = 0; j < kAccItems; ++j) {
       const int idx = threadIdx.x + j * kThreads;
       const int row = idx / 16, gn = n0 + idx % 16;
-      prev[j] = (idx < MT * 256 && row < m && gn < a.n) ? static_cast<const float*>(a.out)[static_cast<long>(row) * a.n + gn] : 0.f;
+      const bool live = idx < MT * 256 && row < m && gn < a.n;
+      prev[j] = live ? static_cast<const float*>(a.out)[static_cast<long>(row) * a.n + gn] : 0.f;
+      if (a.bias != nullptr && live) prev[j] += a.bias[gn];
     }
   }
 
@@ -234,7 +240,7 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
             for (int i = 0; i < kAhead; ++i) ss += part[i];      // (in ascending order; a part that is not there adds 0)
           }
         };
-        if ((U == 4 || EPI == kSwigluBf16) && m <= 8) chain(std::integral_constant<int, 16>{});
+        if ((U == 4 || gated(EPI)) && m <= 8) chain(std::integral_constant<int, 16>{});
         else chain(std::integral_constant<int, 4>{});
       }
       part_sum[j0][row] = ss;
@@ -436,7 +442,7 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
     for (int r = 0; r < 4; ++r) red[wave][t][4 * grp + r][col] = acc[t][r];
   __syncthreads();
 
-  constexpr bool kPaired = EPI == kSwigluBf16 || EPI == kRopeKvBf16;   // columns nl and nl + 8 belong together
+  constexpr bool kPaired = gated(EPI) || EPI == kRopeKvBf16;   // columns nl and nl + 8 belong together
   constexpr int kCols = kPaired ? 8 : 16;
   constexpr int kItems = (MT * 16 * kCols + kThreads - 1) / kThreads;
 #pragma unroll
@@ -494,10 +500,10 @@ __global__ __launch_bounds__(kThreads, (XMODE != kPlain || (MT == 1 && U == 2)) 
         for (int off = 1; off < 16; off <<= 1) sq += __shfl_xor(sq, off, kWave);
         if (nl == 0 && idx < MT * 256 && row < m) a.emit_ssq[static_cast<long>(blockIdx.x) * a.emit_stride + row] = sq;
       }
-    } else if constexpr (EPI == kSwigluBf16) {
+    } else if constexpr (gated(EPI)) {
       // block b = n0 / 16 holds gates and ups of outputs 8b .. 8b + 7
       const long o = static_cast<long>(row) * (a.n / 2) + (n0 / 2 + nl);
-      static_cast<bf16_t*>(a.out)[o] = from_float<bf16_t>(silu_quick(sum) * partner);
+      static_cast<bf16_t*>(a.out)[o] = from_float<bf16_t>((EPI == kGegluBf16 ? gelu_tanh_quick(sum) : silu_quick(sum)) * partner);
     } else {
       const RopeKvArgs& r = a.rope;
       const int d = r.head_dim;
@@ -600,6 +606,7 @@ int launch_epilogue(SkinnyArgs& a, int epilogue, hipStream_t s) {
       if constexpr (XMODE == kPlain) return launch<kAccumF32, XMODE>(a, s);
       else return fail("gemm_skinny: adding into the stream that is being normed is not supported");
     case kSwigluBf16: return launch<kSwigluBf16, XMODE>(a, s);
+    case kGegluBf16: return launch<kGegluBf16, XMODE>(a, s);
     case kRopeKvBf16: return launch<kRopeKvBf16, XMODE>(a, s);
     default: return fail("gemm_skinny: unknown epilogue %d", epilogue);
   }
@@ -608,8 +615,8 @@ int launch_epilogue(SkinnyArgs& a, int epilogue, hipStream_t s) {
 int check_common(const char* what, int m, int max_m, int n, int k, int epilogue) {
   BC4G_REQUIRE(m >= 0 && m <= max_m, "%s: M=%d must be at most %d", what, m, max_m);
   BC4G_REQUIRE(n > 0 && k > 0 && k % 8 == 0, "%s: K=%d must be a positive multiple of 8 (N=%d)", what, k, n);
-  BC4G_REQUIRE(epilogue != kSwigluBf16 || n % 16 == 0,
-               "%s: SwiGLU needs blocks of eight gate and eight up rows, N=%d is no multiple of 16", what, n);
+  BC4G_REQUIRE(!gated(epilogue) || n % 16 == 0,
+               "%s: a gated product needs blocks of eight gate and eight up rows, N=%d is no multiple of 16", what, n);
   return 0;
 }
 
@@ -653,25 +660,28 @@ int check_parts(const char* what, const float* ssq_parts, int ssq_blocks, int ss
 }  // namespace
 }  // namespace bc4g
 
-extern "C" int bc4g_gemm_skinny(const void* x, const void* w, void* out, int epilogue, int m, int n, int k,
+extern "C" int bc4g_gemm_skinny(const void* x, const void* w, void* out, const float* bias, int epilogue, int m, int n, int k,
                                 void* stream) {
   if (int e = check_common("gemm_skinny", m, 64, n, k, epilogue)) return e;
   BC4G_REQUIRE(epilogue != kRopeKvBf16, "gemm_skinny: use bc4g_gemm_skinny_qkv for the rotary epilogue");
+  BC4G_REQUIRE(!bias || epilogue == kAccumF32, "gemm_skinny: only the adding epilogue takes a bias");
   if (m == 0) return 0;
   SkinnyArgs a = plain_args(x, w, out, m, n, k);
+  a.bias = bias;
   return launch_epilogue<kPlain>(a, epilogue, static_cast<hipStream_t>(stream));
 }
 
-// out (the float residual stream, [m, n]) += x w^T, and what the RMSNorm after it needs: emit_x
+// out (the float residual stream, [m, n]) += x w^T + bias (null: none), and what the RMSNorm after it needs: emit_x
 // [m, n] = bfloat16(new residual * g) and emit_ssq [ceil(n / 16)][emit_stride], block b's part of
 // every row's sum of squares.
-extern "C" int bc4g_gemm_skinny_emit(const void* x, const void* w, float* out, const void* g, int g_dtype, void* emit_x,
+extern "C" int bc4g_gemm_skinny_emit(const void* x, const void* w, float* out, const float* bias, const void* g, int g_dtype, void* emit_x,
                                      float* emit_ssq, int emit_stride, int m, int n, int k, void* stream) {
   if (int e = check_common("gemm_skinny_emit", m, 64, n, k, kAccumF32)) return e;
   BC4G_REQUIRE(g && emit_x && emit_ssq && emit_stride >= m, "gemm_skinny_emit: the norm's scale and both outputs are needed");
   BC4G_REQUIRE(g_dtype == kBF16 || g_dtype == kF32, "gemm_skinny_emit: unknown norm scale dtype %d", g_dtype);
   if (m == 0) return 0;
   SkinnyArgs a = plain_args(x, w, out, m, n, k);
+  a.bias = bias;
   a.emit_g = g;
   a.emit_g_f32 = g_dtype == kF32 ? 1 : 0;
   a.emit_x = static_cast<bf16_t*>(emit_x);

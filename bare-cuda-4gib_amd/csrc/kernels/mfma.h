@@ -33,6 +33,12 @@ __device__ inline float silu_quick(float x) {
   return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f));
 }
 
+// z (1 + tanh(u)) / 2 = z / (1 + e^(-2u)) with u = sqrt(2 / pi) (z + 0.044715 z^3), by the same two instructions.
+__device__ inline float gelu_tanh_quick(float z) {
+  const float u2 = z * fmaf(z * z, 2.0f * 0.7978845608028654f * 0.044715f, 2.0f * 0.7978845608028654f);
+  return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(u2 * -1.4426950408889634f));
+}
+
 __device__ inline uint4 load16(const void* p) { return *reinterpret_cast<const uint4*>(p); }
 __device__ inline uint4 zero16() { return make_uint4(0u, 0u, 0u, 0u); }
 

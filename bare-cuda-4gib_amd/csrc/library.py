@@ -23,11 +23,11 @@ _SIGNATURES = {
     "bc4g_rmsnorm_groups": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P],
     "bc4g_stream_update": [_P, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _I, _F, _P],
     "bc4g_embed_beside": [_P, _P, _I, _P, _F, _P, _I, _I, _I, _I, _P],
-    "bc4g_rmsnorm_sum": [_P, _P, _I, _P, _I, _P, _I, _I, _I, _F, _P],
+    "bc4g_rmsnorm_sum": [_P, _P, _I, _P, _P, _I, _P, _I, _I, _I, _F, _P],
     "bc4g_gemm_mfma_parts": [_P, _P, _I, _P, _I, _I, _I, _I, _P],
-    "bc4g_gemm_mfma_swiglu_scaled": [_P, _P, _I, _I, _F, _P, _I, _P, _I, _I, _I, _P],
-    "bc4g_gemm_generic": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _P],
-    "bc4g_swiglu": [_P, _P, _I, _I, _I, _I, _P],
+    "bc4g_gemm_mfma_swiglu_scaled": [_P, _P, _I, _I, _F, _P, _I, _P, _I, _I, _I, _I, _P],
+    "bc4g_gemm_generic": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _I, _I, _P],
+    "bc4g_swiglu": [_P, _P, _I, _I, _I, _I, _I, _P],
     "bc4g_rope_table": [_P, _P, _I, _I, _F, _P],
     "bc4g_rope_kv_write_blocks": [_P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "bc4g_rope_kv_write": [_P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P],
@@ -38,14 +38,14 @@ _SIGNATURES = {
     "bc4g_argmax_static": [_P, _P, _I, _I, _P],
     "bc4g_probe_read": [_P, c_long, _P, _I, _P],
     "bc4g_probe_mfma": [_P, _I, _P, _I, _P],
-    "bc4g_gemm_skinny": [_P, _P, _P, _I, _I, _I, _I, _P],
-    "bc4g_gemm_mfma": [_P, _P, _I, _P, _I, _I, _I, _I, _P],
+    "bc4g_gemm_skinny": [_P, _P, _P, _P, _I, _I, _I, _I, _P],
+    "bc4g_gemm_mfma": [_P, _P, _I, _P, _P, _I, _I, _I, _I, _P],
     "bc4g_gemm_mfma_tile": [_P, _P, _I, _I, _I, _I, _P, _P],
     "bc4g_gemm_skinny_normed": [_P, _P, _P, _I, _F, _P, _P, _I, _I, _I, _I, _P],
     "bc4g_attention_mfma": [_P, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P, _I, _P, _I, _P, _P],
     "bc4g_gemm_mfma_qkv": [_P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "bc4g_gemm_skinny_qkv": [_P, _P, _I, _F, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
-    "bc4g_gemm_skinny_emit": [_P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _P],
+    "bc4g_gemm_skinny_emit": [_P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _P],
     "bc4g_gemm_skinny_prenormed": [_P, _P, _I, _I, _F, _P, _P, _I, _I, _I, _I, _P],
     "bc4g_rmsnorm_add": [_P, _P, _I, _P, _I, _I, _F, _P],
     "bc4g_xielu": [_P, _P, _I, _P, c_long, _P],
@@ -53,8 +53,8 @@ _SIGNATURES = {
     "bc4g_causal_conv": [_P, _I, _P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, c_long, _P],
     "bc4g_rglru_scan": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, c_long, _P],
     "bc4g_latent_angles": [_P, _P, _I, _I, _F, _P],
-    "bc4g_latent_prepare": [_P, _P, _I, _P, _F, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, c_long, c_long, _P],
-    "bc4g_heads_gemm": [_P, _I, c_long, c_long, _P, _I, _P, _I, c_long, c_long, _I, _I, _I, _I, _P],
+    "bc4g_latent_prepare": [_P, _P, _I, _P, _F, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, c_long, c_long, _I, _P, _P, _P, _I, c_long, _P],
+    "bc4g_heads_gemm": [_P, _I, c_long, c_long, _P, _I, _P, _I, c_long, c_long, _I, _I, _I, _I, _P, _I, c_long, _P],
     "bc4g_attention_latent": [_P, _P, _P, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _P],
     "bc4g_clamped_glu": [_P, _P, _I, _F, _F, _I, _I, _P],
     "bc4g_streams_read": [_P, _P, _P, _P, _P, _P, _F, _P, _I, _I, _I, _I, _P],
@@ -66,8 +66,10 @@ _SIGNATURES = {
     "bc4g_heads_finish": [_P, _P, _F, _F, _P, _I, c_long, _I, _P, _I, _I, _I, _I, _P],
     "bc4g_decay_scan": [_P, _I, c_long, _F, _P, _I, c_long, _P, _I, c_long, _P, _P, _I, c_long, _P, _F, _P, _P, _P, _P, _P, _P, _P,
                         _I, _I, _I, _I, _I, _I, _P],
+    "bc4g_matrix_memory": [_P, _P, _P, _P, _P, _P, _I, c_long, _P, _P, _F, _F, _P, _F, _F, _P, _I, c_long, _P, _P, _P, _P, _P, _P, _P,
+                           _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "bc4g_attention_maps": [_P, c_long, _P, _P, _I, _P, _I, _P, _P, _F, _I, _F, _F, _P, _I, c_long, _I, _P, _I,
-                            _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P, _I, _F, _P, _P],
+                            c_long, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P, _I, _F, _P, _P],
     "bc4g_attention_talk": [_P, c_long, _P, _P, _I, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, c_long, _P, _I,
                             _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P, c_long, _P],
     "bc4g_embed_add": [_P, _I, _P, _P, _I, _I, _I, _P],

@@ -18,6 +18,7 @@ from ..errors import KernelError
 from . import library
 
 F32, BF16 = 0, 1
+_GLU_ACT = {"silu": 0, "gelu_tanh": 1}      # the activations of a gated unit's gate
 _CODE = {torch.float32: F32, torch.bfloat16: BF16}
 
 
@@ -216,11 +217,12 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.
 
 
 def gemm_generic(a: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype = None,
-                 accumulate_into: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 accumulate_into: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """a [M, K] times w [N, K] transposed, in plain float arithmetic.  With
-    ``accumulate_into`` (float32 [M, N]) the product is added to it in place."""
+    ``accumulate_into`` (float32 [M, N]) the product is added to it in place, and with it ``bias`` (float32 [N])."""
     w = _rows(w)
-    _dev("gemm", a, w, accumulate_into)
+    _dev("gemm", a, w, accumulate_into, bias)
+    _check_bias("gemm", bias, w.shape[0], accumulate_into)
     if a.dim() != 2 or w.dim() != 2 or a.shape[1] != w.shape[1]:
         raise KernelError(f"gemm: shapes {tuple(a.shape)} x {tuple(w.shape)}^T do not match")
     m, k = a.shape
@@ -232,14 +234,19 @@ def gemm_generic(a: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype = None
     else:
         out = torch.empty((m, n), dtype=out_dtype or a.dtype, device=a.device)
     library.call("bc4g_gemm_generic", _ptr(a), _code(a, "gemm"), _ptr(w), _code(w, "gemm"), _ptr(out),
-                 _code(out, "gemm"), 1 if accumulate_into is not None else 0, m, n, k, _stream(),
+                 _code(out, "gemm"), 1 if accumulate_into is not None else 0, _ptr(bias), m, n, k, _stream(),
                  cost=_gemm_cost(m, n, k, a.element_size(), w.element_size(),
                                  8 if accumulate_into is not None else out.element_size()))
     return out
 
 
-def swiglu(gu: torch.Tensor, interleaved: bool = False) -> torch.Tensor:
-    """gu [T, 2I] -> silu(gate) * up, [T, I].  gu holds all gates then all ups, or (interleaved)
+def _check_bias(what: str, bias: Optional[torch.Tensor], n: int, accumulate_into: Optional[torch.Tensor]) -> None:
+    if bias is not None and (accumulate_into is None or bias.dtype != torch.float32 or tuple(bias.shape) != (n,)):
+        raise KernelError(f"{what}: a bias is float32 [{n}] and joins a product that is added to something, got {bias.dtype} {tuple(bias.shape)}")
+
+
+def swiglu(gu: torch.Tensor, interleaved: bool = False, act: str = "silu") -> torch.Tensor:
+    """gu [T, 2I] -> silu(gate) * up, [T, I] (``act`` "gelu_tanh": the gelu written with tanh for the silu).  gu holds all gates then all ups, or (interleaved)
     blocks of 16: eight gates and the eight ups of the same outputs."""
     _dev("swiglu", gu)
     if gu.dim() != 2 or gu.shape[1] % 2:
@@ -248,7 +255,7 @@ def swiglu(gu: torch.Tensor, interleaved: bool = False) -> torch.Tensor:
     out = torch.empty((t, inter), dtype=gu.dtype, device=gu.device)
     if interleaved and inter % 8:
         raise KernelError(f"swiglu: the interleaved layout needs I={inter} to be a multiple of 8")
-    library.call("bc4g_swiglu", _ptr(gu), _ptr(out), _code(gu, "swiglu"), t, inter, 1 if interleaved else 0, _stream(),
+    library.call("bc4g_swiglu", _ptr(gu), _ptr(out), _code(gu, "swiglu"), t, inter, 1 if interleaved else 0, _GLU_ACT[act], _stream(),
                  cost=lambda: (4.0 * t * inter, 3 * t * inter * gu.element_size()))
     return out
 
@@ -651,6 +658,13 @@ def streams_weights(m: int, n: int, k: int) -> bool:
 
 EPI_STORE_BF16, EPI_STORE_F32, EPI_ACCUM_F32, EPI_SWIGLU = 0, 1, 2, 3
 EPI_SQUARED_RELU = 6      # max(sum, 0)^2 stored as bfloat16
+EPI_GEGLU = 7             # as EPI_SWIGLU, with the gelu written with tanh
+GATED_EPILOGUES = (EPI_SWIGLU, EPI_GEGLU)
+
+
+def gated_epilogue(act: str) -> int:
+    """The epilogue of a gate-up product whose gate goes through ``act`` ("silu" or "gelu_tanh")."""
+    return GATED_EPILOGUES[_GLU_ACT[act]]
 
 
 def _fast_operands(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -659,16 +673,18 @@ def _fast_operands(a: torch.Tensor, w: torch.Tensor) -> bool:
 
 
 def gemm_fast(a: torch.Tensor, w, out_dtype=None,
-              accumulate_into: Optional[torch.Tensor] = None, squared_relu: bool = False) -> Optional[torch.Tensor]:
+              accumulate_into: Optional[torch.Tensor] = None, squared_relu: bool = False,
+              bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """The matrix-core product where a kernel takes these operands (bfloat16, k a multiple of
     8), else None (the caller then uses the plain float kernel).  Up to 64 rows the weights
     are streamed once (a decode step); a wide output goes to the tiled kernel from 24 rows on,
     everything from 65.  ``squared_relu``: the result is max(product, 0)^2, applied to the float sums
-    inside the product's kernel (a bfloat16 result only)."""
+    inside the product's kernel (a bfloat16 result only).  ``bias`` (float32 [n]): added with an adding product."""
     w, packed = _weight(w)
     if not _fast_operands(a, w) or (squared_relu and (accumulate_into is not None or (out_dtype or a.dtype) != torch.bfloat16)):
         return None
-    _dev("gemm", a, w, accumulate_into)
+    _dev("gemm", a, w, accumulate_into, bias)
+    _check_bias("gemm", bias, w.shape[0], accumulate_into)
     m, k = a.shape
     n = w.shape[0]
     if accumulate_into is not None:
@@ -686,10 +702,10 @@ def gemm_fast(a: torch.Tensor, w, out_dtype=None,
         packed = packed if packed is not None else pack_weight(_rows(w))      # (packing per call: tests only)
         for r0 in range(0, m, SKINNY_MAX_ROWS):                        # the weights once for every 64 rows
             rows = min(SKINNY_MAX_ROWS, m - r0)
-            library.call("bc4g_gemm_skinny", _ptr(a[r0:]), _ptr(packed), _ptr(out[r0:]), epi, rows, n, k, _stream(),
+            library.call("bc4g_gemm_skinny", _ptr(a[r0:]), _ptr(packed), _ptr(out[r0:]), _ptr(bias), epi, rows, n, k, _stream(),
                          cost=_skinny_cost(rows, n, k, 2, out_bytes))
     else:
-        library.call("bc4g_gemm_mfma", _ptr(a), *_tiled_weight(w, packed, a), _ptr(out), epi, m, n, k, _stream(),
+        library.call("bc4g_gemm_mfma", _ptr(a), *_tiled_weight(w, packed, a), _ptr(out), _ptr(bias), epi, m, n, k, _stream(),
                      cost=_tiled_cost(m, n, k, out_bytes))
     return out
 
@@ -710,7 +726,7 @@ def gemm_normed_supported(x: torch.Tensor, n_rows: int, g: torch.Tensor, w) -> b
 def gemm_normed(x: torch.Tensor, rows: Optional[torch.Tensor], n_rows: int, g: torch.Tensor, eps: float,
                 w, epilogue: int) -> torch.Tensor:
     """rmsnorm(x[rows]) W^T with the norm fused into the product (see gemm_skinny.hip): epilogue
-    EPI_STORE_BF16, EPI_STORE_F32, EPI_SQUARED_RELU or EPI_SWIGLU (w = gate rows then up rows)."""
+    EPI_STORE_BF16, EPI_STORE_F32, EPI_SQUARED_RELU or a gated one (w in blocks of eight gate and eight up rows)."""
     w, packed = _weight(w)
     packed = packed if packed is not None else pack_weight(_rows(w))
     _dev("gemm_normed", x, rows, g, w)
@@ -721,7 +737,7 @@ def gemm_normed(x: torch.Tensor, rows: Optional[torch.Tensor], n_rows: int, g: t
         _i32("gemm_normed", "rows", rows, n_rows)
     elif n_rows != x.shape[0]:
         raise KernelError("gemm_normed: without row indices every row of x is used")
-    if epilogue == EPI_SWIGLU:
+    if epilogue in GATED_EPILOGUES:
         out = torch.empty((n_rows, n // 2), dtype=torch.bfloat16, device=x.device)
     elif epilogue in (EPI_STORE_BF16, EPI_SQUARED_RELU):
         out = torch.empty((n_rows, n), dtype=torch.bfloat16, device=x.device)
@@ -735,8 +751,8 @@ def gemm_normed(x: torch.Tensor, rows: Optional[torch.Tensor], n_rows: int, g: t
     return out
 
 
-def gemm_swiglu(a: torch.Tensor, w_gate_up, interleaved: bool = False) -> torch.Tensor:
-    """silu(a Wg^T) * (a Wu^T), [M, I], for w_gate_up [2I, K].  interleaved: every 16 rows of the
+def gemm_swiglu(a: torch.Tensor, w_gate_up, interleaved: bool = False, act: str = "silu") -> torch.Tensor:
+    """silu(a Wg^T) * (a Wu^T), [M, I], for w_gate_up [2I, K] (``act`` "gelu_tanh": that gelu for the silu).  interleaved: every 16 rows of the
     weight are eight gate rows and the eight up rows of the same outputs -- then the activation
     is applied to the float sums inside the product's kernel.  Otherwise the product is stored
     and the activation kernel follows."""
@@ -750,16 +766,16 @@ def gemm_swiglu(a: torch.Tensor, w_gate_up, interleaved: bool = False) -> torch.
             packed = packed if packed is not None else pack_weight(_rows(rows))
             for r0 in range(0, m, SKINNY_MAX_ROWS):
                 part = min(SKINNY_MAX_ROWS, m - r0)
-                library.call("bc4g_gemm_skinny", _ptr(a[r0:]), _ptr(packed), _ptr(out[r0:]), EPI_SWIGLU, part, n, k,
+                library.call("bc4g_gemm_skinny", _ptr(a[r0:]), _ptr(packed), _ptr(out[r0:]), None, gated_epilogue(act), part, n, k,
                              _stream(), cost=_skinny_cost(part, n, k, 2, 1))
         else:
-            library.call("bc4g_gemm_mfma", _ptr(a), *_tiled_weight(rows, packed, a), _ptr(out), EPI_SWIGLU, m, n, k, _stream(),
+            library.call("bc4g_gemm_mfma", _ptr(a), *_tiled_weight(rows, packed, a), _ptr(out), None, gated_epilogue(act), m, n, k, _stream(),
                          cost=_tiled_cost(m, n, k, 1))
         return out
     gu = gemm_fast(a, w_gate_up, a.dtype)
     if gu is None:
         gu = gemm_generic(a, w_gate_up, a.dtype)
-    return swiglu(gu, interleaved)
+    return swiglu(gu, interleaved, act)
 
 
 class Fresh:
@@ -806,13 +822,14 @@ def gemm_parts_supported(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Te
 
 
 def gemm_parts_accumulate_norm(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Tensor, eps: float,
-                               checked: bool = False) -> Finished:
-    """residual += a w^T and the RMSNorm (scale g, eps) of the result, in two kernels: the tiled product with k cut
+                               checked: bool = False, bias: Optional[torch.Tensor] = None) -> Finished:
+    """residual += a w^T (+ ``bias``, float32 [n]) and the RMSNorm (scale g, eps) of the result, in two kernels: the tiled product with k cut
     into parts over workgroups, each part's sums stored apart; then one that adds the parts to the residual in
     order and norms it.  For a few dozen rows and a square or long weight, where a 64 x 64 tile's workgroup
     would walk all of k alone and the weight-streaming kernel's workgroups all read all of x."""
     w, packed = _weight(w)
-    _dev("gemm_parts_accumulate_norm", a, w, residual, g)
+    _dev("gemm_parts_accumulate_norm", a, w, residual, g, bias)
+    _check_bias("gemm_parts_accumulate_norm", bias, w.shape[0], residual)
     m, k = a.shape
     n = w.shape[0]
     n_parts = parts_of_k(m, n, k)
@@ -822,7 +839,7 @@ def gemm_parts_accumulate_norm(a: torch.Tensor, w, residual: torch.Tensor, g: to
     out = torch.empty((m, n), dtype=torch.bfloat16, device=a.device)
     library.call("bc4g_gemm_mfma_parts", _ptr(a), *_tiled_weight(w, packed), _ptr(parts), m, n, k, n_parts, _stream(),
                  cost=_gemm_cost(m, n, k, 2, 2, 4 * n_parts, x_readers=-(-n // 64), w_readers=-(-m // 64)))
-    library.call("bc4g_rmsnorm_sum", _ptr(residual), _ptr(parts), n_parts, _ptr(g), _code(g, "rmsnorm_sum"), _ptr(out),
+    library.call("bc4g_rmsnorm_sum", _ptr(residual), _ptr(parts), n_parts, _ptr(bias), _ptr(g), _code(g, "rmsnorm_sum"), _ptr(out),
                  _code(out, "rmsnorm_sum"), m, n, float(eps), _stream(),
                  cost=lambda: (3.0 * m * n + n_parts * m * n, m * n * (4 * n_parts + 8 + 2) + n * g.element_size()))
     return Finished(out)
@@ -836,11 +853,13 @@ def gemm_emit_supported(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Ten
             and g.dtype in _CODE and tuple(g.shape) == (w.shape[0],))
 
 
-def gemm_accumulate_emit(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Tensor, eps: float) -> Prenormed:
-    """residual += a w^T, and the next RMSNorm (scale g, eps) prepared: see Prenormed."""
+def gemm_accumulate_emit(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Tensor, eps: float,
+                         bias: Optional[torch.Tensor] = None) -> Prenormed:
+    """residual += a w^T (+ ``bias``, float32 [n]), and the next RMSNorm (scale g, eps) prepared: see Prenormed."""
     w, packed = _weight(w)
     packed = packed if packed is not None else pack_weight(_rows(w))
-    _dev("gemm_accumulate_emit", a, w, residual, g)
+    _dev("gemm_accumulate_emit", a, w, residual, g, bias)
+    _check_bias("gemm_accumulate_emit", bias, w.shape[0], residual)
     m, k = a.shape
     n = w.shape[0]
     if tuple(residual.shape) != (m, n) or residual.dtype != torch.float32 or not residual.is_contiguous():
@@ -851,7 +870,7 @@ def gemm_accumulate_emit(a: torch.Tensor, w, residual: torch.Tensor, g: torch.Te
     parts = torch.empty((-(-n // 16), m), dtype=torch.float32, device=a.device)
     for r0 in range(0, m, SKINNY_MAX_ROWS):
         rows = min(SKINNY_MAX_ROWS, m - r0)
-        library.call("bc4g_gemm_skinny_emit", _ptr(a[r0:]), _ptr(packed), _ptr(residual[r0:]), _ptr(g),
+        library.call("bc4g_gemm_skinny_emit", _ptr(a[r0:]), _ptr(packed), _ptr(residual[r0:]), _ptr(bias), _ptr(g),
                      _code(g, "gemm_accumulate_emit"), _ptr(xb[r0:]), _ptr(parts[:, r0:]), m, rows, n, k, _stream(),
                      cost=_skinny_cost(rows, n, k, 2, 10))
     return Prenormed(xb, parts, eps)
@@ -867,20 +886,20 @@ def gemm_prenormed_supported(pre: Prenormed, w, epilogue: Optional[int] = None) 
     if not _fast_operands(pre.xb, w):
         return False
     m, (n, k) = pre.xb.shape[0], w.shape
-    return streams_weights(m, n, k) or (epilogue == EPI_SWIGLU and tiled_takes_prenormed(m, n, k)
+    return streams_weights(m, n, k) or (epilogue in GATED_EPILOGUES and tiled_takes_prenormed(m, n, k)
                                         and _ptr(pre.xb) % 16 == 0 and _ptr(w) % 16 == 0)
 
 
 def gemm_prenormed(pre: Prenormed, w, epilogue: int) -> torch.Tensor:
     """rmsnorm(residual) w^T from what gemm_accumulate_emit left: epilogue EPI_STORE_BF16,
-    EPI_STORE_F32, EPI_SQUARED_RELU or EPI_SWIGLU (w in blocks of eight gate and eight up rows)."""
+    EPI_STORE_F32, EPI_SQUARED_RELU or a gated one (w in blocks of eight gate and eight up rows)."""
     w, packed = _weight(w)
     tiled_w = _tiled_weight(w, packed)
     packed = packed if packed is not None else pack_weight(_rows(w))
     _dev("gemm_prenormed", pre.xb, pre.parts, w)
     m, k = pre.xb.shape
     n = w.shape[0]
-    if epilogue == EPI_SWIGLU:
+    if epilogue in GATED_EPILOGUES:
         out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=w.device)
     elif epilogue in (EPI_STORE_BF16, EPI_SQUARED_RELU):
         out = torch.empty((m, n), dtype=torch.bfloat16, device=w.device)
@@ -889,10 +908,10 @@ def gemm_prenormed(pre: Prenormed, w, epilogue: int) -> torch.Tensor:
     else:
         raise KernelError(f"gemm_prenormed: epilogue {epilogue} is not supported")
     if not streams_weights(m, n, k):
-        if epilogue != EPI_SWIGLU:
-            raise KernelError("gemm_prenormed: the tiled kernel finishes a prepared norm in its SwiGLU epilogue only")
+        if epilogue not in GATED_EPILOGUES:
+            raise KernelError("gemm_prenormed: the tiled kernel finishes a prepared norm in its gated epilogues only")
         library.call("bc4g_gemm_mfma_swiglu_scaled", _ptr(pre.xb), _ptr(pre.parts), pre.parts.shape[0], pre.parts.shape[1], pre.eps,
-                     *tiled_w, _ptr(out), m, n, k, _stream(), cost=_tiled_cost(m, n, k, 1))
+                     *tiled_w, _ptr(out), 1 if epilogue == EPI_GEGLU else 0, m, n, k, _stream(), cost=_tiled_cost(m, n, k, 1))
         return out
     for r0 in range(0, m, SKINNY_MAX_ROWS):
         rows = min(SKINNY_MAX_ROWS, m - r0)
@@ -1430,39 +1449,53 @@ def latent_angles(positions: torch.Tensor, dims: int, base: float) -> torch.Tens
     return table
 
 
-def latent_prepare(q: torch.Tensor, dkv: Optional[torch.Tensor], g: Optional[torch.Tensor], eps: float, angles: Optional[torch.Tensor],
-                   slot_map: Optional[torch.Tensor], cache: Optional[torch.Tensor], q_lat: torch.Tensor, heads: int, plain: int,
-                   rot: int, rank: int, dims: int) -> None:
+def latent_prepare(q: Optional[torch.Tensor], dkv: Optional[torch.Tensor], g: Optional[torch.Tensor], eps: float, angles: Optional[torch.Tensor],
+                   slot_map: Optional[torch.Tensor], cache: Optional[torch.Tensor], q_lat: Optional[torch.Tensor], heads: int, plain: int,
+                   rot: int, rank: int, dims: int, *, halves: bool = False, low: Optional[torch.Tensor] = None,
+                   low_g: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """Writes [rmsnorm(dkv[:, :rank]) * g | rotate(dkv[:, rank:])] into every row's cache slot (``cache`` None: nowhere)
     and every head's rotated query part into q_lat[:, h, rank:].  ``angles``: latent_angles of the rows (None where
-    nothing is rotated, dims 0).  Without a cache dkv and g may be None: only the queries are rotated."""
-    _dev("latent_prepare", g, angles, slot_map, cache, q_lat)
-    if cache is None and rot == 0:
-        return                  # nothing to write
-    q_row = _rows_of("latent_prepare", "q", q)                 # (q and dkv may be parts of one product's rows)
-    dkv_row = _rows_of("latent_prepare", "dkv", dkv) if dkv is not None else 0
-    t = q.shape[0]
-    if tuple(q.shape) != (t, heads * (plain + rot)) or (dkv is not None and (q.dtype != dkv.dtype or tuple(dkv.shape) != (t, rank + rot))):
-        raise KernelError(f"latent_prepare: q {tuple(q.shape)} / dkv {tuple(dkv.shape) if dkv is not None else None} do not fit "
-                          f"heads={heads} plain={plain} rot={rot} rank={rank}")
+    nothing is rotated, dims 0).  Without a cache dkv and g may be None: only the queries are rotated.  ``halves``: element
+    i of the first dims turns with element i + dims / 2 (else neighbours turn together).  ``low`` [T, low_rank]: the queries'
+    own latent; returns rmsnorm(low) * low_g (the same eps), from which they are made -- q and q_lat are None then."""
+    _dev("latent_prepare", g, angles, slot_map, cache, q_lat, low_g)
+    if cache is None and (rot == 0 or q is None) and low is None:
+        return None             # nothing to write
+    some = next(x for x in (q, dkv, low) if x is not None)
+    t = some.shape[0]
+    # (q, dkv and low may be parts of one product's rows)
+    q_row, dkv_row, low_row = (_rows_of("latent_prepare", name, x) if x is not None else 0 for name, x in (("q", q), ("dkv", dkv), ("low", low)))
+    if ((q is None) != (q_lat is None) or (q is not None and tuple(q.shape) != (t, heads * (plain + rot)))
+            or (dkv is not None and (some.dtype != dkv.dtype or tuple(dkv.shape) != (t, rank + rot)))
+            or (low is not None and (some.dtype != low.dtype or low.shape[0] != t or low_g is None))):
+        raise KernelError(f"latent_prepare: q {tuple(q.shape) if q is not None else None} / dkv {tuple(dkv.shape) if dkv is not None else None} / "
+                          f"low {tuple(low.shape) if low is not None else None} do not fit heads={heads} plain={plain} rot={rot} rank={rank}")
     _f32("latent_prepare", "g", g, (rank,))
     _f32("latent_prepare", "q_lat", q_lat, (t, heads, rank + rot))
+    low_rank = low.shape[1] if low is not None else 0
+    _f32("latent_prepare", "low_g", low_g, (low_rank,))
+    low_out = torch.empty((t, low_rank), dtype=low.dtype, device=low.device) if low is not None else None
     if dims:
         _f32("latent_prepare", "angles", angles, (t, dims // 2, 2))
     if cache is not None:
         if dkv is None or g is None:
             raise KernelError("latent_prepare: a cache row is made of dkv and g")
-        if cache.dtype != q.dtype or cache.dim() != 3 or cache.shape[2] != rank + rot:
-            raise KernelError(f"latent_prepare: the cache must be {q.dtype} [pages, page_tokens, {rank + rot}], got {cache.dtype} {tuple(cache.shape)}")
+        if cache.dtype != some.dtype or cache.dim() != 3 or cache.shape[2] != rank + rot:
+            raise KernelError(f"latent_prepare: the cache must be {some.dtype} [pages, page_tokens, {rank + rot}], got {cache.dtype} {tuple(cache.shape)}")
         _i32("latent_prepare", "slot_map", slot_map, t)
-    library.call("bc4g_latent_prepare", _ptr(q), _ptr(dkv), _code(q, "latent_prepare"), _ptr(g), float(eps),
+    turned = (heads if q is not None else 0) + (1 if cache is not None else 0)
+    normed = (rank if cache is not None else 0) + low_rank
+    library.call("bc4g_latent_prepare", _ptr(q), _ptr(dkv), _code(some, "latent_prepare"), _ptr(g), float(eps),
                  _ptr(angles) if dims else None, _ptr(slot_map) if cache is not None else None, _ptr(cache), _ptr(q_lat), t, heads,
-                 plain, rot, rank, int(dims), q_row, dkv_row, _stream(), cost=lambda: (4.0 * t * (rank + (heads + 1) * rot), t * (q.element_size() * (heads + 2) * rot + 2 * rank * q.element_size())))
+                 plain, rot, rank, int(dims), q_row, dkv_row, 1 if halves else 0, _ptr(low), _ptr(low_g), _ptr(low_out), low_rank, low_row,
+                 _stream(), cost=lambda: (4.0 * t * (normed + turned * rot), t * some.element_size() * ((turned + 1) * rot + 2 * normed)))
+    return low_out
 
 
-def heads_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, k: int, n: int) -> None:
+def heads_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, k: int, n: int, gate: Optional[torch.Tensor] = None) -> None:
     """out[t, h, :n] = w[h] a[t, h, :k] for a [T, heads, >= k], w [heads, n, k], out [T, heads, >= n] (the last
-    dimensions may be longer than k and n: parts of wider rows)."""
+    dimensions may be longer than k and n: parts of wider rows).  ``gate`` [T, heads] (may be a part of wider rows): head h's
+    outputs are multiplied by sigmoid(gate[t, h])."""
     _dev("heads_gemm", w, out)
     if a.dim() != 3 or out.dim() != 3 or w.dim() != 3 or a.shape[:2] != out.shape[:2] or a.shape[2] < k or out.shape[2] < n \
             or tuple(w.shape) != (a.shape[1], n, k):
@@ -1470,8 +1503,12 @@ def heads_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, k: int, n: i
     if not a.is_cuda or a.stride(2) != 1 or a.stride(1) < k or a.stride(0) < a.stride(1):      # (a's rows may be parts of wider rows)
         raise KernelError(f"heads_gemm: a must lie on the GPU with a head's elements side by side, got strides {a.stride()}")
     t, heads = a.shape[0], a.shape[1]
+    gate_row = _part_of_rows("heads_gemm", "gate", gate, heads) if gate is not None else 0
+    if gate is not None and gate.shape[0] != t:
+        raise KernelError(f"heads_gemm: gate has {gate.shape[0]} rows, a {t}")
     library.call("bc4g_heads_gemm", _ptr(a), _code(a, "heads_gemm"), a.stride(0), a.stride(1), _ptr(w), _code(w, "heads_gemm"),
-                 _ptr(out), _code(out, "heads_gemm"), heads * out.shape[2], out.shape[2], t, n, k, heads, _stream(),
+                 _ptr(out), _code(out, "heads_gemm"), heads * out.shape[2], out.shape[2], t, n, k, heads, _ptr(gate),
+                 _code(gate, "heads_gemm") if gate is not None else F32, gate_row, _stream(),
                  cost=lambda: (2.0 * t * heads * n * k, heads * n * k * w.element_size() + t * heads * (k * a.element_size() + n * out.element_size())))
 
 
@@ -1625,6 +1662,16 @@ def _part_of_rows(what: str, name: str, t: torch.Tensor, width: int) -> int:
     return t.stride(0)
 
 
+def _place_for(what: str, out: Optional[torch.Tensor], rows: int, width: int, dtype: torch.dtype, device):
+    """(tensor [rows, width], elements from row to row) a result goes to: a new one, or ``out``, which may be a part of wider rows."""
+    if out is None:
+        return torch.empty((rows, width), dtype=dtype, device=device), width
+    stride = _part_of_rows(what, "out", out, width)
+    if tuple(out.shape) != (rows, width) or out.dtype != dtype:
+        raise KernelError(f"{what}: out must be {dtype} [{rows}, {width}], got {out.dtype} {tuple(out.shape)}")
+    return out, stride if rows > 1 else max(stride, width)
+
+
 def rotary_table(positions: torch.Tensor, freqs: torch.Tensor, amplitude: float = 1.0) -> torch.Tensor:
     """[T, half, 2] float32: cos and sin of positions[t] * freqs[i] (freqs float64 [half] on the device), times
     ``amplitude``; the angles are worked out in double."""
@@ -1646,18 +1693,21 @@ class _PrepareSection(ctypes.Structure):
                 ("page_stride", ctypes.c_long), ("head_stride", ctypes.c_long), ("token_stride", ctypes.c_long),
                 ("in_dtype", ctypes.c_int), ("out_dtype", ctypes.c_int), ("half", ctypes.c_int), ("page_tokens", ctypes.c_int),
                 ("heads", ctypes.c_int), ("dim", ctypes.c_int), ("eps", ctypes.c_float), ("factor", ctypes.c_float),
-                ("pairing", ctypes.c_int), ("unit_after", ctypes.c_int), ("norm_rows", ctypes.c_int)]
+                ("pairing", ctypes.c_int), ("unit_after", ctypes.c_int), ("norm_rows", ctypes.c_int), ("temp_coef", ctypes.c_float),
+                ("temp_every", ctypes.c_double), ("positions", ctypes.c_void_p)]
 
 
 def heads_section(x: torch.Tensor, heads: int, dim: int, out: torch.Tensor, *, bias: Optional[torch.Tensor] = None,
                   norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0, table: Optional[torch.Tensor] = None,
                   factor: float = 1.0, slot_map: Optional[torch.Tensor] = None, page_tokens: int = 0,
-                  neighbours: bool = False, unit_after: bool = False, norm_rows: bool = False):
+                  neighbours: bool = False, unit_after: bool = False, norm_rows: bool = False,
+                  temperature: Optional[Tuple[torch.Tensor, float, float]] = None):
     """One section for heads_prepare_many: every head of x [T, heads * dim] (may be a part of wider rows): + bias, RMS norm
     over the head with ``norm_weight`` [dim], rotation by ``table`` [T, half, 2] (element i with element i + half, or with
     ``neighbours`` element 2i with element 2i + 1), with ``unit_after`` division by sqrt(mean(head^2) + eps) of the head as
     it stands then, times ``factor``.  With ``norm_rows`` the norm before the rotation is taken over the whole row, all heads
-    at once, and ``norm_weight`` is [heads * dim].  ``out``: [T, heads, dim] (float32 or bfloat16), or with ``slot_map`` a cache
+    at once, and ``norm_weight`` is [heads * dim].  ``temperature`` = (positions int32 [T], coef, every): last, a factor
+    1 + coef ln(floor((position + 1) / every) + 1).  ``out``: [T, heads, dim] (float32 or bfloat16), or with ``slot_map`` a cache
     [pages, heads, page_tokens, dim] whose slot page * page_tokens + offset receives the row.  Checked here; the tensors
     must live until the launch."""
     _dev("heads_prepare", bias, norm_weight, table, out, slot_map)
@@ -1681,10 +1731,16 @@ def heads_section(x: torch.Tensor, heads: int, dim: int, out: torch.Tensor, *, b
             raise KernelError(f"heads_prepare: out must be [{t}, {heads}, {dim}], got {tuple(out.shape)}")
         page_stride = head_stride = token_stride = 0
         out_row = heads * dim
+    where, coef, every = temperature if temperature is not None else (None, 0.0, 0.0)
+    if where is not None:
+        _dev("heads_prepare", where)
+        _i32("heads_prepare", "positions", where, t)
+        if every <= 0:
+            raise KernelError(f"heads_prepare: a temperature that grows every {every} positions")
     section = _PrepareSection(_ptr(x), _ptr(bias), _ptr(norm_weight), _ptr(table), _ptr(out), _ptr(slot_map), in_row, out_row,
                               page_stride, head_stride, token_stride, _code(x, "heads_prepare"), _code(out, "heads_prepare"), half,
                               page_tokens, heads, dim, float(eps), float(factor), 1 if neighbours else 0, 1 if unit_after else 0,
-                              1 if norm_rows and norm_weight is not None else 0)
+                              1 if norm_rows and norm_weight is not None else 0, float(coef), float(every), _ptr(where))
     return section, t, t * heads * dim, x.element_size() + out.element_size()
 
 
@@ -1782,12 +1838,63 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.T
     return out
 
 
+def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, zi: torch.Tensor, zf: torch.Tensor, state, ctx,
+                  heads: int, dim: int, vdim: int, *, bias_i: torch.Tensor, bias_f: torch.Tensor, cap: float, weight: torch.Tensor,
+                  eps: float, out_dtype: torch.dtype, factor: float = 1.0, chunk_base: Optional[torch.Tensor] = None, n_chunks: int = 0,
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A matrix memory per request and head over a step's rows (see csrc/kernels/matrix_memory.hip for the equations): q, k
+    [T, heads * dim], v, gate [T, heads * vdim], gate logits zi, zf [T, heads] -- all parts of one tensor's rows --, log gates capped by ``cap``
+    with ``bias_i``, ``bias_f`` (float32 [heads]); q is scaled by dim^(-1/2).  ``state`` = (S [slots, heads, dim, vdim], n [slots, heads,
+    dim], m [slots, heads]), float32, is read and left.  Every head's output is divided by its root mean square (``eps``), times
+    ``weight`` (float32 [heads * vdim]), sigmoid(gate) and ``factor``: [T, heads * vdim], into ``out`` if given (a part of wider rows, say).
+    ``chunk_base`` and ``n_chunks``: as for decay_scan."""
+    S, n, m = state
+    _dev("matrix_memory", bias_i, bias_f, weight, S, n, m, chunk_base)
+    t = q.shape[0]
+    rows = [_part_of_rows("matrix_memory", name, x, width) for name, x, width in
+            (("q", q, heads * dim), ("k", k, heads * dim), ("v", v, heads * vdim), ("gate", gate, heads * vdim), ("zi", zi, heads), ("zf", zf, heads))]
+    if len(set(rows)) != 1 or len({x.dtype for x in (q, k, v, gate, zi, zf)}) != 1 or any(x.shape[0] != t for x in (k, v, gate, zi, zf)):
+        raise KernelError("matrix_memory: q, k, v, the gate and the gates' logits must be parts of one tensor's rows")
+    if dim > HEADS_MAX_DIM or vdim > HEADS_MAX_DIM or cap <= 0:
+        raise KernelError(f"matrix_memory: heads of {dim} x {vdim} (at most {HEADS_MAX_DIM}), gates capped by {cap}")
+    _f32("matrix_memory", "bias_i", bias_i, (heads,))
+    _f32("matrix_memory", "bias_f", bias_f, (heads,))
+    _f32("matrix_memory", "weight", weight, (heads * vdim,))
+    slots = S.shape[0]
+    _f32("matrix_memory", "S", S, (slots, heads, dim, vdim))
+    _f32("matrix_memory", "n", n, (slots, heads, dim))
+    _f32("matrix_memory", "m", m, (slots, heads))
+    if max(ctx.seq_slots, default=0) >= slots:
+        raise KernelError(f"matrix_memory: the state has {slots} slots, the step names slot {max(ctx.seq_slots)}")
+    _check_grouping("matrix_memory", ctx, t)
+    most = max(int(ctx.seq_start[s + 1] - ctx.seq_start[s]) for s in range(ctx.n_seqs))
+    gates = chunk_S = chunk_n = chunk_decay = None
+    if most > DECAY_SCAN_CHUNK:
+        if chunk_base is None or n_chunks < 2:
+            raise KernelError("matrix_memory: a request brings several chunks of rows and the chunks' places are not given")
+        _i32("matrix_memory", "chunk_base", chunk_base, ctx.n_seqs)
+        f32 = dict(dtype=torch.float32, device=S.device)
+        gates = torch.empty((3, t, heads), **f32)
+        chunk_S, chunk_n, chunk_decay = (torch.empty((n_chunks, heads, *rest), **f32) for rest in ((dim, vdim), (dim,), ()))
+    out, out_row = _place_for("matrix_memory", out, t, heads * vdim, out_dtype, S.device)
+    passes = 2 if most > DECAY_SCAN_CHUNK else 1
+    library.call("bc4g_matrix_memory", _ptr(q), _ptr(k), _ptr(v), _ptr(gate), _ptr(zi), _ptr(zf), _code(q, "matrix_memory"), rows[0], _ptr(bias_i),
+                 _ptr(bias_f), float(cap), float(dim) ** -0.5, _ptr(weight), float(eps), float(factor), _ptr(out), _code(out, "matrix_memory"),
+                 out_row, _ptr(S), _ptr(n), _ptr(m), _ptr(gates), _ptr(chunk_S), _ptr(chunk_n), _ptr(chunk_decay), _ptr(ctx.seq_start_dev),
+                 _ptr(ctx.seq_slots_dev), _ptr(chunk_base), t, ctx.n_seqs, most, heads, dim, vdim, _stream(),
+                 cost=lambda: (passes * 4.0 * t * heads * dim * vdim,
+                               t * heads * (2 * dim + 2 * vdim + 2) * q.element_size() + t * heads * vdim * out.element_size()
+                               + 8.0 * ctx.n_seqs * heads * dim * (vdim + 1)))
+    return out
+
+
 def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, ctx, out_dtype: torch.dtype,
                    n_heads: int, n_kv_heads: int, maps: int, dim: int, vdim: int, window: int, keep_first: int, scale: float, *,
                    lam: float = 0.0, normalize: bool = False, eps: float = 0.0, factor: float = 1.0,
                    gate: Optional[torch.Tensor] = None, act: int = ACT_SIGMOID, waves: int = 0,
                    sink: Optional[torch.Tensor] = None, far: Optional[Tuple[torch.Tensor, torch.Tensor]] = None,
-                   block: int = 0, cap: float = 0.0, point: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   block: int = 0, cap: float = 0.0, point: Optional[torch.Tensor] = None,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Softmax attention with ``maps`` (1 or 2) score maps per query head over the same values: q float32
     [T, n_heads, maps, dim]; keys [pages, n_kv_heads * maps, page_tokens, dim], values [pages, n_kv_heads, page_tokens, vdim].
     A row at position p sees key j <= p if p - j < window or j < keep_first (window 0: every key).  o = a1 - lam a2,
@@ -1797,7 +1904,8 @@ def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     no key and no value.  ``far`` = (r1, r2), float32 [n_heads] each: r1 ln(1 + r2 (p - j)) is taken off the scaled score.
     ``block`` (instead of a window): a row sees the keys j <= p of its own block of that many positions, counted from 0.
     ``cap``: the scaled score becomes cap tanh(score / cap).  ``point`` (float32 [n_heads], no sink then): no softmax -- a
-    visible key weighs sigmoid(score + point[head]), nothing is normalised over keys."""
+    visible key weighs sigmoid(score + point[head]), nothing is normalised over keys.  ``out``: where the result goes
+    ([T, n_heads * vdim] in ``out_dtype``, may be a part of wider rows) instead of a tensor of its own."""
     _dev("attention_maps", q, k_cache, v_cache, block_table, sink, point, *(far or ()))
     _f32("attention_maps", "sink", sink, (n_heads,))
     _f32("attention_maps", "point", point, (n_heads,))
@@ -1820,7 +1928,7 @@ def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     _i32("attention_maps", "row_seq", ctx.row_seq, t)
     _i32("attention_maps", "positions", ctx.positions, t)
     gate_row = _part_of_rows("attention_maps", "gate", gate, n_heads * vdim) if gate is not None else 0
-    out = torch.empty((t, n_heads * vdim), dtype=out_dtype, device=q.device)
+    out, out_row = _place_for("attention_maps", out, t, n_heads * vdim, out_dtype, q.device)
 
     def cost():
         keys = pairs = 0
@@ -1844,7 +1952,7 @@ def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     library.call("bc4g_attention_maps", _ptr(q), n_heads * maps * dim, _ptr(k_cache), _ptr(v_cache), _code(k_cache, "attention_maps"),
                  _ptr(block_table), block_table.stride(0), _ptr(ctx.row_seq), _ptr(ctx.positions), float(lam), 1 if normalize else 0,
                  float(eps), float(factor), _ptr(gate), _code(gate, "attention_maps") if gate is not None else F32, gate_row, int(act),
-                 _ptr(out), _code(out, "attention_maps"), t, n_heads, n_kv_heads, maps, dim, vdim, page_tokens, int(window),
+                 _ptr(out), _code(out, "attention_maps"), out_row, t, n_heads, n_kv_heads, maps, dim, vdim, page_tokens, int(window),
                  int(keep_first), float(scale), int(waves), _ptr(sink), _ptr(far[0]) if far else None,
                  _ptr(far[1]) if far else None, int(block), float(cap), _ptr(point), _stream(), cost=cost)
     return out

@@ -122,7 +122,7 @@ bool swiglu() {
       Dev<float> g32(gu), o32(static_cast<size_t>(n) * inter);
       Dev<bf16> g16(as_bf16(gu)), o16(static_cast<size_t>(n) * inter);
       RUN(bc4g_swiglu(dtype ? static_cast<const void*>(g16.p) : g32.p, dtype ? static_cast<void*>(o16.p) : o32.p, dtype, n,
-                      inter, interleaved, kStream));
+                      inter, interleaved, 0, kStream));
       std::vector<double> want;
       for (int t = 0; t < n; ++t)
         for (int i = 0; i < inter; ++i) {
@@ -147,8 +147,8 @@ bool gemm_generic() {
     const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n);
     {   // float x float -> float, and added into a float output
       Dev<float> da(a), dw(w), out(static_cast<size_t>(m) * n), acc(before);
-      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, out.p, 0, 0, m, n, k, kStream));
-      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, acc.p, 0, 1, m, n, k, kStream));
+      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, out.p, 0, 0, nullptr, m, n, k, kStream));
+      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, acc.p, 0, 1, nullptr, m, n, k, kStream));
       const std::vector<double> want = plain::gemm(widen(a), widen(w), m, n, k);
       ok &= close("float product", widen(out.get()), want, 1e-5, 1e-5);
       std::vector<double> sum = want;
@@ -158,7 +158,7 @@ bool gemm_generic() {
     {   // bfloat16 x bfloat16 -> float
       Dev<bf16> da(as_bf16(a)), dw(as_bf16(w));
       Dev<float> out(static_cast<size_t>(m) * n);
-      RUN(bc4g_gemm_generic(da.p, 1, dw.p, 1, out.p, 0, 0, m, n, k, kStream));
+      RUN(bc4g_gemm_generic(da.p, 1, dw.p, 1, out.p, 0, 0, nullptr, m, n, k, kStream));
       ok &= close("bfloat16 product", widen(out.get()), plain::gemm(widen(as_bf16(a)), widen(as_bf16(w)), m, n, k), 1e-5, 1e-5);
     }
   }
@@ -177,12 +177,12 @@ bool gemm_skinny() {
     const std::vector<double> want = plain::gemm(widen(x), widen(w), m, n, k);
     Dev<bf16> dx(x), o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2);
     Dev<float> o32(static_cast<size_t>(m) * n), acc(before);
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, 0, m, n, k, kStream));
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, o32.p, 1, m, n, k, kStream));
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, acc.p, 2, m, n, k, kStream));
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, act.p, 3, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, nullptr, 0, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, o32.p, nullptr, 1, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, acc.p, nullptr, 2, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, act.p, nullptr, 3, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, 6, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, nullptr, 6, m, n, k, kStream));
     std::vector<double> squared = want;
     for (double& v : squared) v = plain::squared_relu(v);
     ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
@@ -231,7 +231,7 @@ bool gemm_skinny_norms() {
   const std::vector<float> residual = normals(rng, static_cast<size_t>(m) * hidden, 2.0f);
   Dev<bf16> dx(x), p1(pack_weight(w1, hidden, k1)), p2(pack_weight(w2, n2, hidden)), emit_x(static_cast<size_t>(m) * hidden);
   Dev<float> dres(residual), ssq(static_cast<size_t>((hidden + 15) / 16) * m), y(static_cast<size_t>(m) * n2);
-  RUN(bc4g_gemm_skinny_emit(dx.p, p1.p, dres.p, dg.p, 0, emit_x.p, ssq.p, m, m, hidden, k1, kStream));
+  RUN(bc4g_gemm_skinny_emit(dx.p, p1.p, dres.p, nullptr, dg.p, 0, emit_x.p, ssq.p, m, m, hidden, k1, kStream));
   RUN(bc4g_gemm_skinny_prenormed(emit_x.p, ssq.p, (hidden + 15) / 16, m, eps, p2.p, y.p, 1, m, n2, hidden, kStream));
   std::vector<double> after = plain::gemm(widen(x), widen(w1), m, hidden, k1);
   for (size_t i = 0; i < after.size(); ++i) after[i] += residual[i];
@@ -248,7 +248,7 @@ bool gemm_skinny_norms() {
   const int n3 = 96;
   const std::vector<bf16> w3 = as_bf16(normals(rng, static_cast<size_t>(n3) * hidden, 0.3f));
   Dev<bf16> p3(pack_weight(w3, n3, hidden)), act(static_cast<size_t>(m) * n3 / 2);
-  RUN(bc4g_gemm_mfma_swiglu_scaled(emit_x.p, ssq.p, (hidden + 15) / 16, m, eps, p3.p, 1, act.p, m, n3, hidden, kStream));
+  RUN(bc4g_gemm_mfma_swiglu_scaled(emit_x.p, ssq.p, (hidden + 15) / 16, m, eps, p3.p, 1, act.p, 0, m, n3, hidden, kStream));
   const std::vector<double> gu = plain::gemm(normed2, widen(w3), m, n3, hidden);
   std::vector<double> gated;
   for (int r = 0; r < m; ++r)
@@ -272,12 +272,12 @@ bool gemm_mfma() {
     const void* dw = w_packed ? packed.p : rows.p;
     Dev<bf16> o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2);
     Dev<float> o32(static_cast<size_t>(m) * n), acc(before);
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, 0, m, n, k, kStream));
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o32.p, 1, m, n, k, kStream));
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, acc.p, 2, m, n, k, kStream));
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, act.p, 3, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, nullptr, 0, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o32.p, nullptr, 1, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, acc.p, nullptr, 2, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, act.p, nullptr, 3, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, 6, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, nullptr, 6, m, n, k, kStream));
     std::vector<double> squared = want;
     for (double& v : squared) v = plain::squared_relu(v);
     ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
@@ -302,7 +302,7 @@ bool gemm_mfma() {
   Dev<bf16> dx(x), pw(pack_weight(wo, width, depth)), normed(static_cast<size_t>(rows_few) * width);
   Dev<float> dparts(static_cast<size_t>(parts) * rows_few * width), dres(residual), dg(g);
   RUN(bc4g_gemm_mfma_parts(dx.p, pw.p, 1, dparts.p, rows_few, width, depth, parts, kStream));
-  RUN(bc4g_rmsnorm_sum(dres.p, dparts.p, parts, dg.p, 0, normed.p, 1, rows_few, width, eps, kStream));
+  RUN(bc4g_rmsnorm_sum(dres.p, dparts.p, parts, nullptr, dg.p, 0, normed.p, 1, rows_few, width, eps, kStream));
   std::vector<double> after = plain::gemm(widen(x), widen(wo), rows_few, width, depth), y;
   for (size_t i = 0; i < after.size(); ++i) after[i] += residual[i];
   ok &= close("stream after the parts were added", widen(dres.get()), after, 1e-4, 1e-4);

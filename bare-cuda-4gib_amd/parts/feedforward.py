@@ -14,13 +14,17 @@ from .linear import linear, linear_squared_relu, linear_swiglu
 
 class SwiGLU(Part):
     """x += (silu(h Wg^T) * (h Wu^T)) Wd^T with silu(g) = g / (1 + exp(-g)), no
-    biases (reference: engine/src/model.cpp:579-603, engine/kernels/swiglu.cu:17-25)."""
+    biases (reference: engine/src/model.cpp:579-603, engine/kernels/swiglu.cu:17-25).  ``act`` "gelu_tanh":
+    g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))) / 2 takes the place of the silu."""
     category = "feedforward"
     graph_safe = True     # launches kernels only: may run inside a captured graph
     accepts_lazy_norm = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int):
+    def __init__(self, hidden_size: int, intermediate_size: int, act: str = "silu"):
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+        if act not in ("silu", "gelu_tanh"):
+            raise ConfigError(f"gated feed-forward: activation {act!r} ('silu' or 'gelu_tanh')")
+        self.act = act
         self.w_gu = self.w_down = None
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
@@ -51,7 +55,7 @@ class SwiGLU(Part):
         return self.interleaved and self.w_gu.plan.wants_prepared(n_rows, swiglu=True)
 
     def forward(self, h, ctx, residual) -> None:
-        act = linear_swiglu(h, self.w_gu, self.interleaved)
+        act = linear_swiglu(h, self.w_gu, self.interleaved, self.act)
         linear(act, self.w_down, accumulate_into=residual, ctx=ctx)
 
 

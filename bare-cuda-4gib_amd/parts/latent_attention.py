@@ -16,9 +16,10 @@ from .linear import linear
 class LatentAttention(Part):
     """Every token keeps a latent c = rmsnorm(Wdkv h [:rank]) * g and one rotated key part kr = rotate(Wdkv h [rank:])
     for all heads; head a's key is [Wuk_a c | kr], its value Wuv_a c, its query [q_plain | rotate(q_rot)] of
-    q = Wq h.  Scores (q . k) * scale over the keys at or before the row's position (within ``window`` if not 0); the
+    q = Wq h (with ``q_rank`` the queries come from a latent of their own: q = Wuq (rmsnorm(Wdq h) * gq)).  Scores (q . k) * scale over the keys at or before the row's position (within ``window`` if not 0); the
     softmax's denominator also holds exp(sink_a) (``sink``: a learned number per head without key or value).
-    Rotation: elements 2i and 2i+1 of the first ``rot_dims`` of a rotated part turn by position * base^(-2i/rot_dims).
+    Rotation: elements 2i and 2i+1 of the first ``rot_dims`` of a rotated part turn by position * base^(-2i/rot_dims), or with
+    ``pairing`` "half" elements i and i + rot_dims/2.  ``head_gate``: head a's output is multiplied by sigmoid(Wg h)_a (``g``).
 
     Only c and kr are cached (cache.specs.PagedLatent).  The keys' up-projection is absorbed into the query
     (Wuk_a^T q_plain scores against c directly) and the values' up-projection is applied to the weighted sum of the
@@ -33,7 +34,8 @@ class LatentAttention(Part):
     accepts_lazy_norm = True  # (one product reads the norm)
 
     def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, kv_rank: int, scale: float, eps: float, rot_dim: int = 0,
-                 rot_dims: int = 0, rot_base: float = 10000.0, sink: bool = True, window: int = 0, borrows: bool = False):
+                 rot_dims: int = 0, rot_base: float = 10000.0, sink: bool = True, window: int = 0, borrows: bool = False,
+                 q_rank: int = 0, pairing: str = "neighbours", head_gate: bool = False):
         for name, v in (("heads", heads), ("dim", dim), ("vdim", vdim), ("kv_rank", kv_rank), ("hidden_size", hidden_size)):
             if int(v) <= 0:
                 raise ConfigError(f"latent attention: {name} must be positive, got {v}")
@@ -41,19 +43,26 @@ class LatentAttention(Part):
             raise ConfigError(f"latent attention: {rot_dims} rotated dimensions (even) of a rotated part of {rot_dim}")
         if rot_base <= 0 or window < 0:
             raise ConfigError(f"latent attention: rotation base {rot_base}, window {window}")
+        if q_rank < 0 or pairing not in ("half", "neighbours"):
+            raise ConfigError(f"latent attention: the queries' latent of {q_rank} numbers, pairing {pairing!r} ('half' or 'neighbours')")
         if kv_rank + rot_dim > ops.LATENT_MAX_ROW:
             raise ConfigError(f"latent attention: kv_rank + rot_dim = {kv_rank + rot_dim} is beyond the kernel's {ops.LATENT_MAX_ROW}")
         self.hidden_size, self.heads, self.dim, self.rot_dim = int(hidden_size), int(heads), int(dim), int(rot_dim)
         self.vdim, self.kv_rank, self.scale, self.rot_dims = int(vdim), int(kv_rank), float(scale), int(rot_dims)
         self.rot_base, self.eps, self.sink, self.window = float(rot_base), float(eps), bool(sink), int(window)
         self.borrows = bool(borrows)
+        self.q_rank, self.halves, self.head_gate = int(q_rank), pairing == "half", bool(head_gate)
 
     def cache_spec(self):
         return PagedLatent(self.kv_rank, self.rot_dim, self.window)
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
         H, w = self.heads, self.hidden_size
-        out = {"q": WeightSpec((H * (self.dim + self.rot_dim), w))}
+        n_q = H * (self.dim + self.rot_dim)
+        out = {"q": WeightSpec((n_q, w))} if not self.q_rank else {
+            "dq": WeightSpec((self.q_rank, w)), "dq.norm": WeightSpec((self.q_rank,), kind="vector", init="ones"), "uq": WeightSpec((n_q, self.q_rank))}
+        if self.head_gate:
+            out["g"] = WeightSpec((H, w))
         if not self.borrows:
             out.update({"dkv": WeightSpec((self.kv_rank + self.rot_dim, w)), "dkv.norm": WeightSpec((self.kv_rank,), kind="vector", init="ones")})
         out.update({"uk": WeightSpec((H * self.dim, self.kv_rank)), "uv": WeightSpec((H * self.vdim, self.kv_rank)),
@@ -64,8 +73,11 @@ class LatentAttention(Part):
 
     def bind(self, tensors, rt) -> None:
         H = self.heads
-        # one product for the queries and the latent: their rows one after the other
-        self.w_qd = ops.StreamedWeight(tensors["q"] if self.borrows else torch.cat([tensors["q"], tensors["dkv"]], dim=0).contiguous())
+        # one product for the queries (or their latent), the latent and the heads' gates: their rows one after the other
+        names = ["dq" if self.q_rank else "q"] + ([] if self.borrows else ["dkv"]) + (["g"] if self.head_gate else [])
+        self.w_qd = ops.StreamedWeight(torch.cat([tensors[n] for n in names], dim=0).contiguous())
+        self.w_uq = ops.StreamedWeight(tensors["uq"]) if self.q_rank else None
+        self.gq = tensors["dq.norm"].to(torch.float32).contiguous() if self.q_rank else None
         self.w_o = ops.StreamedWeight(tensors["o"])
         self.g = None if self.borrows else tensors["dkv.norm"].to(torch.float32).contiguous()
         # [heads, rank, dim]: the keys' up-projection as it is applied to the query
@@ -93,22 +105,28 @@ class LatentAttention(Part):
         H, rank, rot = self.heads, self.kv_rank, self.rot_dim
         if self.borrows and writes:
             raise ConfigError("latent attention: a layer without a latent of its own cannot write a cache stream")
-        n_q = H * (self.dim + rot)
+        n_q = self.q_rank or H * (self.dim + rot)
+        n_kv = 0 if self.borrows else rank + rot
         qd = linear(h, self.w_qd, out_dtype=self.act_dtype)
         t = qd.shape[0]
-        q, dkv = qd[:, :n_q], None if self.borrows else qd[:, n_q:]
+        q, dkv = qd[:, :n_q], None if self.borrows else qd[:, n_q:n_q + n_kv]
+        gate = qd[:, n_q + n_kv:] if self.head_gate else None
         q_lat = torch.empty((t, H, rank + rot), dtype=torch.float32, device=q.device)
         angles = None
         if self.rot_dims:                 # the same in every layer that rotates alike: a table made once a step
             angles = ctx.shared(("latent_angles", self.rot_dims, self.rot_base),
                                 lambda: ops.latent_angles(ctx.positions, self.rot_dims, self.rot_base))
-        ops.latent_prepare(q, dkv, self.g, self.eps, angles, ctx.slot_maps[cache.group] if writes else None,
-                           cache.latent if writes else None, q_lat, H, self.dim, rot, rank, self.rot_dims)
+        where, to = (ctx.slot_maps[cache.group], cache.latent) if writes else (None, None)
+        sizes = (H, self.dim, rot, rank, self.rot_dims)
+        if self.q_rank:           # both latents are normed by one kernel, then the queries are made and turned
+            low = ops.latent_prepare(None, dkv, self.g, self.eps, angles, where, to, None, *sizes, halves=self.halves, low=q, low_g=self.gq)
+            q, dkv, to = linear(low, self.w_uq, out_dtype=self.act_dtype), None, None
+        ops.latent_prepare(q, dkv, self.g, self.eps, angles, where, to, q_lat, *sizes, halves=self.halves)
         ops.heads_gemm(q.unflatten(1, (H, self.dim + rot)), self.uk_t, q_lat, k=self.dim, n=rank)
         mixed = ops.attention_latent(q_lat, cache.latent, self.sinks, ctx.block_tables[cache.group], ctx, H, rank, rot,
                                      cache.page_tokens, self.window, self.scale)
         o = torch.empty((t, H, self.vdim), dtype=self.act_dtype, device=q.device)
-        ops.heads_gemm(mixed, self.uv, o, k=rank, n=self.vdim)
+        ops.heads_gemm(mixed, self.uv, o, k=rank, n=self.vdim, gate=gate)
         linear(o.view(t, H * self.vdim), self.w_o, accumulate_into=residual, ctx=ctx)
 
 

@@ -1,12 +1,13 @@
 """Linear attention with a decayed matrix state per head: retention (a constant decay per head, rotated queries and
-keys) and gated linear attention (a decay per key channel and token, made from the input)."""
+keys), gated linear attention (a decay per key channel and token, made from the input) and a matrix memory (a decay and an
+exponential input gate per head and token, with a normaliser)."""
 from __future__ import annotations
 
 from typing import Dict, Optional, Sequence
 
 import torch
 
-from ..cache.specs import FixedState
+from ..cache.specs import FixedState, States
 from ..csrc import ops
 from ..errors import ConfigError
 from ..weights.loader import WeightSpec
@@ -143,5 +144,69 @@ class GatedLinearAttention(_DecayedState):
                accumulate_into=residual, ctx=ctx)
 
 
+class MatrixMemory(_DecayedState):
+    """q = Wq h dim^(-1/2), k = Wk h (heads x dim), v = Wv h (heads x vdim); per head log gates i = cap tanh((Wi h + bi) / cap) and
+    f = log sigmoid(cap tanh((Wf h + bf) / cap)).  With a running maximum m (from 0), m_t = max(f + m_(t-1), i):
+    S_t = e^(f + m_(t-1) - m_t) S_(t-1) + e^(i - m_t) k v^T, n_t likewise with k alone,
+    o_t = S_t^T q / (max(|n_t . q|, e^(-m_t)) + 1e-6); the head's o divided by its root mean square, the heads side by side times
+    the weight ``norm`` [heads * vdim] and sigmoid(Wg h), projected by Wo.  The product's outputs stay float32: the gates' logits
+    are among them.  The state S, n, m is float32.  A mixer of this kind can stand beside another one (see parts.parallel)."""
+    accepts_lazy_norm = True  # (one product reads the norm)
+    stands_beside = True
+
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, gate_cap: float, eps: float):
+        self._sizes(hidden_size, heads, dim, vdim, "matrix memory")
+        self.gate_cap, self.eps = float(gate_cap), float(eps)
+        if self.gate_cap <= 0:
+            raise ConfigError(f"matrix memory: the gates' cap {gate_cap} must be positive")
+
+    def cache_spec(self):
+        H, d, e = self.heads, self.dim, self.vdim
+        return States((("S", (H, d, e), "float32"), ("n", (H, d), "float32"), ("m", (H,), "float32")))
+
+    def weight_specs(self) -> Dict[str, WeightSpec]:
+        qk, v, h, H = self.heads * self.dim, self.heads * self.vdim, self.hidden_size, self.heads
+        vec = lambda n, init="normal": WeightSpec((n,), kind="vector", init=init)      # noqa: E731
+        return {"q": WeightSpec((qk, h)), "k": WeightSpec((qk, h)), "v": WeightSpec((v, h)), "g": WeightSpec((v, h)), "i": WeightSpec((H, h)),
+                "i.b": vec(H), "f": WeightSpec((H, h)), "f.b": vec(H), "norm": vec(v, "ones"), "o": WeightSpec((h, v))}
+
+    @property
+    def heads_width(self) -> int:
+        return self.heads * self.vdim
+
+    def input_names(self):
+        return ["q", "k", "v", "g", "i", "f"]
+
+    def bind(self, tensors, rt) -> None:
+        self.w_in = ops.StreamedWeight(torch.cat([tensors[n] for n in self.input_names()], dim=0).contiguous())
+        self.w_o = ops.StreamedWeight(tensors["o"])
+        self.bind_heads(tensors, rt)
+
+    def bind_heads(self, tensors, rt) -> None:
+        self.i_b, self.f_b, self.norm_w = (tensors[n].to(torch.float32).contiguous() for n in ("i.b", "f.b", "norm"))
+        self.o_b = None
+        self.act_dtype = rt.act_dtype
+
+    def wants_prepared_norm(self, n_rows: int) -> bool:
+        return self.act_dtype == torch.bfloat16 and self.w_in.plan.wants_prepared(n_rows)
+
+    def forward(self, h, ctx, cache, residual, writes: bool = True) -> None:
+        o = self.run_heads(linear(h, self.w_in, out_dtype=torch.float32), ctx, cache, writes)
+        linear(o, self.w_o, accumulate_into=residual, ctx=ctx)
+
+    def run_heads(self, x, ctx, cache, writes: bool = True, out=None, factor: float = 1.0) -> torch.Tensor:
+        """The heads' outputs side by side [T, heads * vdim], times ``factor``, from the rows x of the input product; into ``out``
+        (a part of wider rows, say) if given."""
+        if not writes:
+            raise ConfigError("matrix memory: a state is moved by every row that reads it")
+        H, d, e = self.heads, self.dim, self.vdim
+        q, k, v, g, zi, zf = torch.split(x, [H * d, H * d, H * e, H * e, H, H], dim=1)
+        base, n_chunks = self._chunks(ctx)
+        return ops.matrix_memory(q, k, v, g, zi, zf, (cache.S, cache.n, cache.m), ctx, H, d, e, bias_i=self.i_b, bias_f=self.f_b,
+                                 cap=self.gate_cap, weight=self.norm_w, eps=self.eps, out_dtype=self.act_dtype, factor=factor,
+                                 chunk_base=base, n_chunks=n_chunks, out=out)
+
+
 register_part("mixer", "retention", Retention)
 register_part("mixer", "gla", GatedLinearAttention)
+register_part("mixer", "matrix_memory", MatrixMemory)

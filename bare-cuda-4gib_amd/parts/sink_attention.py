@@ -43,16 +43,27 @@ class SinkAttention(Part):
                 sequence's first token (wherever a prompt was cut)
     cap         the scaled score becomes cap tanh(score / cap)
     sink        "unit": the sink is the number 1 in every head's denominator, exp(0), and no tensor
-    weights     "sigmoid": no softmax and no sink -- a visible key weighs sigmoid(score + ``pb``[a]) by itself"""
+    weights     "sigmoid": no softmax and no sink -- a visible key weighs sigmoid(score + ``pb``[a]) by itself
+
+    Two more for queries and keys, and one for the output, with any of the above:
+
+    head_norm   every head of q and k RMS-normed with a weight that all heads share (``q.norm`` [dim], ``k.norm`` [dim]), before
+                the rotation
+    temperature (coef, every): queries grow with their position p by a factor 1 + coef ln(1 + floor((p + 1) / every)), applied last
+    out_bias    ``o.b`` is added to the output projection
+
+    A mixer of this kind can stand beside another one (see parts.parallel), unless its projections go through a
+    convolution or its heads mix their weights or carry a gate."""
     category = "mixer"
     graph_safe = True     # launches kernels only: may run inside a captured graph
     adds_one_product = True   # the output is one last product through linear(): a block may hand it ops.Fresh
+    accepts_lazy_norm = True  # (one product reads the norm)
 
     def __init__(self, hidden_size: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float = 0.0,
                  window: int = 0, conv_taps: int = 0, position=None, unit_norm: bool = False, sink: bool = True,
                  distance: bool = False, talking: bool = False, head_gate: bool = False, bias: bool = False,
                  values: str = "projected", row_norm: bool = False, value_unit_norm: bool = False, block: int = 0,
-                 cap: float = 0.0, weights: str = "softmax"):
+                 cap: float = 0.0, weights: str = "softmax", head_norm: bool = False, temperature=None, out_bias: bool = False):
         if values not in ("projected", "keys") or weights not in ("softmax", "sigmoid") or sink not in (True, False, "unit", "learned"):
             raise ConfigError(f"sink attention: values {values!r} ('projected' or 'keys'), weights {weights!r} ('softmax' or "
                               f"'sigmoid'), sink {sink!r} (true, false or 'unit')")
@@ -78,6 +89,12 @@ class SinkAttention(Part):
         self.talking, self.head_gate = bool(talking), bool(head_gate)
         self.bias, self.own_values, self.row_norm = bool(bias), values == "projected", bool(row_norm)
         self.value_unit_norm, self.block, self.cap = bool(value_unit_norm), int(block), float(cap)
+        self.head_norm, self.out_bias = bool(head_norm), bool(out_bias)
+        if self.head_norm and self.row_norm:
+            raise ConfigError("sink attention: queries and keys are normed over the head or over the row, not both")
+        self.temperature = (float(temperature[0]), float(temperature[1])) if temperature is not None else None
+        if self.temperature is not None and self.temperature[1] <= 0:
+            raise ConfigError(f"sink attention: a temperature that grows every {temperature[1]} positions")
         self.position = build_part("position", position) if position is not None else None
         if self.position is not None and not hasattr(self.position, "table"):
             raise ConfigError("sink attention: the position part must give a table of cosines and sines")
@@ -115,6 +132,10 @@ class SinkAttention(Part):
                 out["v.b"] = vec(G * e)
         if self.row_norm:
             out.update({"q.norm": vec(H * d), "k.norm": vec(G * d)})
+        if self.head_norm:
+            out.update({"q.norm": WeightSpec((d,), kind="vector", init="ones"), "k.norm": WeightSpec((d,), kind="vector", init="ones")})
+        if self.out_bias:
+            out["o.b"] = vec(h)
         if self.squash:
             out["pb"] = vec(H)
         if self.conv_taps:
@@ -129,11 +150,25 @@ class SinkAttention(Part):
             out["g"] = WeightSpec((H, h))
         return out
 
+    # ---- what a mixer that can stand beside another one says (parts.parallel) ----
+    @property
+    def stands_beside(self) -> bool:
+        return not self.conv_taps and not self.together
+
+    @property
+    def heads_width(self) -> int:
+        return self.heads * self.vdim
+
+    def input_names(self):
+        return ["q", "k"] + (["v"] if self.own_values else []) + (["g"] if self.head_gate else [])
+
     def bind(self, tensors, rt) -> None:
-        f32 = lambda name: tensors[name].to(torch.float32).contiguous()      # noqa: E731
-        names = ["q", "k"] + (["v"] if self.own_values else []) + (["g"] if self.head_gate else [])
-        self.w_in = ops.StreamedWeight(torch.cat([tensors[n] for n in names], dim=0).contiguous())
+        self.w_in = ops.StreamedWeight(torch.cat([tensors[n] for n in self.input_names()], dim=0).contiguous())
         self.w_o = ops.StreamedWeight(tensors["o"])
+        self.bind_heads(tensors, rt)
+
+    def bind_heads(self, tensors, rt) -> None:
+        f32 = lambda name: tensors[name].to(torch.float32).contiguous()      # noqa: E731
         self.conv_w = None
         if self.conv_taps:      # by taps, the channels of q, k and v side by side as in the product's rows
             self.conv_w = torch.cat([f32(n + ".conv") for n in ("q", "k", "v")], dim=0).t().contiguous()
@@ -143,7 +178,8 @@ class SinkAttention(Part):
         self.point_w = f32("pb") if self.squash else None
         self.q_b, self.k_b = (f32("q.b"), f32("k.b")) if self.bias else (None, None)
         self.v_b = (f32("v.b") if self.own_values else self.k_b) if self.bias else None
-        self.q_norm, self.k_norm = (f32("q.norm"), f32("k.norm")) if self.row_norm else (None, None)
+        self.q_norm, self.k_norm = (f32("q.norm"), f32("k.norm")) if self.row_norm or self.head_norm else (None, None)
+        self.o_b = f32("o.b") if self.out_bias else None
         self.far = (f32("r1"), f32("r2")) if self.distance else None
         self.talk_w = f32("talk") if self.talking else None
         self.act_dtype = rt.act_dtype
@@ -176,9 +212,19 @@ class SinkAttention(Part):
     def working_bytes_per_row(self, elem: int) -> float:
         return super().working_bytes_per_row(elem) + self.channels * elem + self.heads * (4 * self.dim + self.vdim * elem)
 
+    def wants_prepared_norm(self, n_rows: int) -> bool:
+        """Whether the first product is better served by a norm that the product before prepared than by fusing the
+        norm or running it: the weight's own plan says (ops.LinearPlan.wants_prepared)."""
+        return self.act_dtype == torch.bfloat16 and self.w_in.plan.wants_prepared(n_rows)
+
     def forward(self, h, ctx, cache, residual, writes: bool = True) -> None:
-        H, G, d, e, t = self.heads, self.kv_heads, self.dim, self.vdim, h.shape[0]
-        x = linear(h, self.w_in, out_dtype=self.act_dtype)
+        o = self.run_heads(linear(h, self.w_in, out_dtype=self.act_dtype), ctx, cache, writes)
+        linear(o, self.w_o, accumulate_into=residual, ctx=ctx, bias=self.o_b)
+
+    def run_heads(self, x, ctx, cache, writes: bool = True, out=None, factor: float = 1.0) -> torch.Tensor:
+        """The heads' outputs side by side [T, heads * vdim], times ``factor``, from the rows x of the input product; into ``out``
+        (a part of wider rows, say) if given."""
+        H, G, d, e, t = self.heads, self.kv_heads, self.dim, self.vdim, x.shape[0]
         nq, nk, nv = H * d, G * d, G * e
         gate = x[:, nq + nk + nv:] if self.head_gate else None
         kv = cache
@@ -194,7 +240,8 @@ class SinkAttention(Part):
                     norm_rows=self.row_norm)
         q_heads = torch.empty((t, H, d), dtype=torch.float32, device=x.device)
         # queries dense in float32, keys and values straight into their pages: one launch for the three
-        sections = [ops.heads_section(q, H, d, q_heads, bias=self.q_b, norm_weight=self.q_norm, **turn)]
+        temperature = (ctx.positions, *self.temperature) if self.temperature is not None else None
+        sections = [ops.heads_section(q, H, d, q_heads, bias=self.q_b, norm_weight=self.q_norm, temperature=temperature, **turn)]
         if writes:
             slots = ctx.slot_maps[kv.group]
             sections.append(ops.heads_section(k, G, d, kv.k, slot_map=slots, page_tokens=kv.page_tokens, bias=self.k_b,
@@ -203,13 +250,11 @@ class SinkAttention(Part):
                                               unit_after=self.value_unit_norm, eps=self.eps))
         ops.heads_prepare_many(sections)
         if self.together:
-            o = ops.attention_talk(q_heads, kv.k, kv.v, ctx.block_tables[kv.group], ctx, self.act_dtype, H, G, d, e, self.window,
-                                   self.scale, sink=self.sink_w, far=self.far, talk=self.talk_w, gate=gate)
-        else:
-            o = ops.attention_maps(q_heads.view(t, H, 1, d), kv.k, kv.v, ctx.block_tables[kv.group], ctx, self.act_dtype, H, G, 1,
-                                   d, e, self.window, 0, self.scale, sink=self.sink_w, far=self.far, block=self.block, cap=self.cap,
-                                   point=self.point_w)
-        linear(o, self.w_o, accumulate_into=residual, ctx=ctx)
+            return ops.attention_talk(q_heads, kv.k, kv.v, ctx.block_tables[kv.group], ctx, self.act_dtype, H, G, d, e, self.window,
+                                      self.scale, sink=self.sink_w, far=self.far, talk=self.talk_w, gate=gate)
+        return ops.attention_maps(q_heads.view(t, H, 1, d), kv.k, kv.v, ctx.block_tables[kv.group], ctx, self.act_dtype, H, G, 1,
+                                  d, e, self.window, 0, self.scale, sink=self.sink_w, far=self.far, block=self.block, cap=self.cap,
+                                  point=self.point_w, out=out, factor=factor)
 
 
 register_part("mixer", "sink_attention", SinkAttention)
