@@ -11,8 +11,9 @@
 //
 // As in decay_scan.hip a request's rows are walked in chunks of 32, a workgroup each, a thread keeping one column of S in
 // registers (the workgroup has a thread for every column, so that a head's root mean square is taken where its values
-// are made); the first wave also keeps n, its channels spread over the lanes.  A request of one chunk (a decode step, a
-// short portion) is one launch, from and into its slot.  Longer ones: the gates of all rows (m is a scan over pairs
+// are made); the first wave also keeps n, its channels spread over the lanes.  A request of one chunk (a short portion) is
+// one launch, from and into its slot; a step in which every request brings one row (decoding) is one launch of a kernel of
+// its own, whose threads share a state's channels too, a few pieces of 16 bytes each.  Longer requests: the gates of all rows (m is a scan over pairs
 // (A, B), m -> max(m + A, B)), every chunk from nothing (what it adds, the product of its decays), the states between the
 // chunks, then every chunk again from its true state, writing outputs.
 #include <math.h>
@@ -309,6 +310,102 @@ __global__ void memory_between_kernel(const MemoryArgs a) {
   *slot = st;
 }
 
+// A step of one row a request: a workgroup a (request, head), its threads in groups of whole rows of S -- thread t takes VEC
+// neighbouring columns and every n_groups-th channel --, so that all of a state's memory is asked for at once.
+constexpr int kStepThreads = 512;
+template <int VEC>
+__global__ __launch_bounds__(kStepThreads) void memory_step_kernel(const MemoryArgs a) {
+  __shared__ float part_s[kStepThreads * VEC];
+  __shared__ float red_s[kStepThreads / kWave];
+  __shared__ float scratch[16];
+  constexpr int kAhead = 8;
+  const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+  const int s = blockIdx.x / a.heads, head = blockIdx.x % a.heads, dim = a.dim, vdim = a.vdim;
+  const long row = a.seq_start[s], slot = static_cast<long>(a.seq_slots[s]) * a.heads + head;
+  const int cols = vdim / VEC, groups = kStepThreads / cols, group = tid / cols, c0 = (tid % cols) * VEC;
+  const bool mine = group < groups;
+  float* S = a.S + slot * dim * vdim;
+  const long at_k = row * a.row + static_cast<long>(head) * dim, at_v = row * a.row + static_cast<long>(head) * vdim;
+
+  // Pieces of the state and the keys and queries that go with them; the first are on their way while the gates are made.
+  float have[kAhead][VEC], kk[kAhead], qq[kAhead];
+  auto fetch = [&](int d0) {
+#pragma unroll
+    for (int b = 0; b < kAhead; ++b) {
+      const int d = d0 + b * groups;
+      const bool ok = mine && d < dim;
+      const float* from = S + static_cast<long>(ok ? d : 0) * vdim + (ok ? c0 : 0);
+      if constexpr (VEC == 4) {
+        const float4 x = *reinterpret_cast<const float4*>(from);
+        have[b][0] = x.x, have[b][1] = x.y, have[b][2] = x.z, have[b][3] = x.w;
+      } else {
+        have[b][0] = *from;
+      }
+      kk[b] = load_any(a.k, a.dtype, at_k + (ok ? d : 0));
+      qq[b] = load_any(a.q, a.dtype, at_k + (ok ? d : 0));
+    }
+  };
+  fetch(group);
+  float v[VEC];
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) v[e] = mine ? load_any(a.v, a.dtype, at_v + c0 + e) : 0.f;
+  float i, f;
+  log_gates(a, row, head, i, f);
+  const float m_in = a.m[slot], m = fmaxf(f + m_in, i);
+  const float dec = expf(f + m_in - m), add = expf(i - m);
+
+  float dot = 0.f;
+  for (int d = tid; d < dim; d += kStepThreads) {
+    const float nd = fmaf(dec, a.n[slot * dim + d], add * load_any(a.k, a.dtype, at_k + d));
+    a.n[slot * dim + d] = nd;
+    dot = fmaf(nd, load_any(a.q, a.dtype, at_k + d) * a.q_scale, dot);
+  }
+  dot = wave_sum(dot);
+  if (lane == 0) red_s[wave] = dot;
+
+  float o[VEC];
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) o[e] = 0.f;
+  for (int d0 = group; d0 < dim; d0 += groups * kAhead) {
+    if (d0 != group) fetch(d0);
+#pragma unroll
+    for (int b = 0; b < kAhead; ++b) {
+      const int d = d0 + b * groups;
+      if (!mine || d >= dim) continue;
+      const float k = add * kk[b], q = a.q_scale * qq[b];
+      float now[VEC];
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        now[e] = fmaf(dec, have[b][e], k * v[e]);
+        o[e] = fmaf(now[e], q, o[e]);
+      }
+      float* to = S + static_cast<long>(d) * vdim + c0;
+      if constexpr (VEC == 4) *reinterpret_cast<float4*>(to) = make_float4(now[0], now[1], now[2], now[3]);
+      else to[0] = now[0];
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < VEC; ++e)
+    if (mine) part_s[group * vdim + c0 + e] = o[e];
+  __syncthreads();
+  if (tid == 0) a.m[slot] = m;                        // (every thread has read the old one)
+  float total = 0.f;
+  for (int w = 0; w < kStepThreads / kWave; ++w) total += red_s[w];
+  const float den = fmaxf(fabsf(total), expf(-m)) + 1e-6f;
+  float val = 0.f;
+  if (tid < vdim) {
+    for (int g = 0; g < groups; ++g) val += part_s[g * vdim + tid];
+    val /= den;
+  }
+  const float by = a.factor / sqrtf(block_sum(val * val, scratch) / static_cast<float>(vdim) + a.eps);
+  if (tid < vdim) {
+    const long col = static_cast<long>(head) * vdim + tid;
+    const float y = val * by * a.weight[col] / (1.0f + expf(-load_any(a.gate, a.dtype, row * a.row + col)));
+    if (a.out_dtype == kF32) static_cast<float*>(a.out)[row * a.out_row + col] = y;
+    else static_cast<bf16_t*>(a.out)[row * a.out_row + col] = from_float<bf16_t>(y);
+  }
+}
+
 template <int KD>
 void launch_memory(const MemoryArgs& a, int n_seqs, int most_chunks, hipStream_t s) {
   dim3 grid(most_chunks, n_seqs * a.heads), block(ceil_div(a.vdim, kWave) * kWave);
@@ -347,6 +444,11 @@ extern "C" int bc4g_matrix_memory(const void* q, const void* k, const void* v, c
   const MemoryArgs a{q, k, v, gate, zi, zf, row, dtype, bi, bf, weight, cap, q_scale, eps, factor, out, out_dtype, out_row,
                      S, n, m, gates, chunk_S, chunk_n, chunk_decay, seq_start, seq_slots, chunk_base, n_rows, heads, dim, vdim};
   hipStream_t s = static_cast<hipStream_t>(stream);
+  if (most_rows == 1) {
+    if (vdim % 4 == 0 && reinterpret_cast<uintptr_t>(S) % 16 == 0) memory_step_kernel<4><<<n_seqs * heads, kStepThreads, 0, s>>>(a);
+    else memory_step_kernel<1><<<n_seqs * heads, kStepThreads, 0, s>>>(a);
+    return check_launch("matrix_memory");
+  }
   if (dim <= 16) launch_memory<16>(a, n_seqs, most_chunks, s);
   else if (dim <= 32) launch_memory<32>(a, n_seqs, most_chunks, s);
   else if (dim <= 64) launch_memory<64>(a, n_seqs, most_chunks, s);

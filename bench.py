@@ -34,7 +34,7 @@ if ROOT not in sys.path:
 
 HBM_PEAK_GBS = 8000.0                       # MI355X: 8 TB/s
 PEAK_TFLOPS = {"bf16": 2500.0, "fp32": 157.3}
-FP32_WORK = {"attention_maps", "attention_talk", "decay_scan"}    # kernels whose arithmetic is float32 by their design's rule
+FP32_WORK = {"attention_maps", "attention_talk", "decay_scan", "matrix_memory"}    # kernels whose arithmetic is float32 by their design's rule
 TINYLLAMA = dict(architectures=["LlamaForCausalLM"], model_type="llama", vocab_size=32000, hidden_size=2048,
                  num_hidden_layers=22, num_attention_heads=32, num_key_value_heads=4, head_dim=64,
                  intermediate_size=5632, rope_theta=10000.0, rms_norm_eps=1e-5,
@@ -171,6 +171,32 @@ BASELIX_SIZES = {
     "1k": (baselix_shape(1024, 6, 8, 64, 64, 256, 4096, 8, 2, 896), MAMENEX_SIZES["1k"][0], MILENEX_SIZES["1k"][0]),
     "2k": (baselix_shape(2048, 6, 16, 128, 128, 512, 8192, 8, 2, 1792), MAMENEX_SIZES["2k"][0], MILENEX_SIZES["2k"][0]),
     "4k": (baselix_shape(4096, 6, 32, 128, 128, 512, 14336, 8, 2, 3200), MAMENEX_SIZES["4k"][0], MILENEX_SIZES["4k"][0]),
+}
+
+
+def varolix_shape(width, layers, heads, kv_heads, dim, vdim, m_heads, m_dim, latent, q_rank, kv_rank, ff, vocab=32000):
+    """A Varolix configuration of real layer sizes: attention beside a matrix memory (m_heads states of m_dim x m_dim), plain
+    attention and latent attention in turn, all with the gated gelu feed-forward; the fourth layer runs twice."""
+    mlp = dict(kind="dense", ff=ff)
+    two = dict(type="parallel", mlp=mlp, mixer=dict(
+        left=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, q_temp=dict(coef=0.1, every=1024)), left_scale=0.7,
+        right=dict(heads=m_heads, dim=m_dim, vdim=m_dim, gate_cap=15.0), right_scale=0.9))
+    one = dict(type="attention", mlp=mlp, mixer=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, rot=dict(
+        base=10000.0, dims=dim // 2, scaling=dict(factor=4.0, original=4096, fast=24.0, slow=2.0))))
+    lat = dict(type="latent_attention", mlp=mlp, mixer=dict(
+        heads=heads, dim=latent, rot_dim=latent // 2, vdim=latent, q_rank=q_rank, kv_rank=kv_rank, scale=(1.5 * latent) ** -0.5,
+        rot=dict(base=10000.0, dims=latent // 2)))
+    order = [(two, one, lat)[i % 3] for i in range(layers)]
+    return dict(architecture="Varolix", vocab=vocab, width=width, norm=dict(eps=1e-6), loop=dict(start=3, stop=4, times=2), layers=order)
+
+
+# --only varolix: the design at a few sizes that resemble a real model's layers (five layers, six layer runs), each beside
+# the Nagezen decoder (the other design here with float32 attention heads, matrix states and gated feed-forwards of the
+# same size) and the Mamenex decoder (latent attention) of the same width, number of layer runs and head count.
+VAROLIX_SIZES = {
+    "1k": (varolix_shape(1024, 5, 8, 2, 64, 128, 4, 128, 64, 384, 224, 2752), NAGEZEN_SIZES["1k"][0], MAMENEX_SIZES["1k"][0]),
+    "2k": (varolix_shape(2048, 5, 16, 4, 64, 128, 8, 128, 128, 768, 512, 5504), NAGEZEN_SIZES["2k"][0], MAMENEX_SIZES["2k"][0]),
+    "4k": (varolix_shape(4096, 5, 32, 8, 64, 128, 16, 128, 128, 1536, 512, 9600), NAGEZEN_SIZES["4k"][0], MAMENEX_SIZES["4k"][0]),
 }
 BASELINE_DECODE_B1 = 77.3                   # the reference's only FP16 decode number (batch 1, RTX 3050)
 
@@ -344,7 +370,7 @@ def kernel_table(model, cfg, prefill_tokens, batch, context, dtype):
 
 def run_mamenex(size, args, only="mamenex", names=("mamenex", "llama"), sizes=None):
     """Prefill and decode of a design at one size beside another decoder of equal size (Mamenex beside Llama, Nagezen
-    beside Mamenex, Milenex beside Nagezen, Lagusun beside Milenex, Baselix beside Mamenex and Milenex); with --kernels the
+    beside Mamenex, Milenex beside Nagezen, Lagusun beside Milenex, Baselix beside Mamenex and Milenex, Varolix beside Nagezen and Mamenex); with --kernels the
     per-kernel tables of all."""
     dtype = "bfloat16" if args.dtype == "bf16" else "float32"
     elem = 2 if args.dtype == "bf16" else 4
@@ -513,9 +539,9 @@ def main() -> int:
     ap.add_argument("--top-p", type=float, default=1.0, help="--only serve: ... and this top-p (1: none)")
     ap.add_argument("--gather-ms", type=float, default=0.0,
                     help="--only chat: the scheduler waits this long before it admits those who came while others decode")
-    ap.add_argument("--sizes", default="1k,2k,4k", help="--only mamenex, nagezen, milenex, lagusun, baselix: which of the sizes " + ", ".join(MAMENEX_SIZES))
-    ap.add_argument("--kernels", action="store_true", help="--only mamenex, nagezen, milenex, lagusun, baselix: add the per-kernel tables (time, part of the roofline)")
-    ap.add_argument("--only", choices=["decode", "prefill", "serve", "chat", "gemm", "peaks", "mamenex", "nagezen", "milenex", "lagusun", "baselix"], default=None,
+    ap.add_argument("--sizes", default="1k,2k,4k", help="--only mamenex, nagezen, milenex, lagusun, baselix, varolix: which of the sizes " + ", ".join(MAMENEX_SIZES))
+    ap.add_argument("--kernels", action="store_true", help="--only mamenex, nagezen, milenex, lagusun, baselix, varolix: add the per-kernel tables (time, part of the roofline)")
+    ap.add_argument("--only", choices=["decode", "prefill", "serve", "chat", "gemm", "peaks", "mamenex", "nagezen", "milenex", "lagusun", "baselix", "varolix"], default=None,
                     help="run one part only and print its own short line (for profiling); peaks: what a kernel that only "
                          "reads, and one of nothing but matrix-core instructions, reach on this device")
     ap.add_argument("--mnk", default="2048,11264,2048",
@@ -551,6 +577,10 @@ def main() -> int:
     if args.only == "baselix":
         for size in args.sizes.split(","):
             print(json.dumps(run_mamenex(size, args, "baselix", ("baselix", "mamenex", "milenex"), BASELIX_SIZES)), flush=True)
+        return 0
+    if args.only == "varolix":
+        for size in args.sizes.split(","):
+            print(json.dumps(run_mamenex(size, args, "varolix", ("varolix", "nagezen", "mamenex"), VAROLIX_SIZES)), flush=True)
         return 0
     from bare_cuda_4gib_amd.csrc.peaks import measured_peaks
     measured = measured_peaks()

@@ -133,17 +133,20 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, i: torch.Te
 # --- the model ---------------------------------------------------------------------
 
 class PlainVarolix:
-    def __init__(self, folder: str, dtype: torch.dtype = torch.float64):
+    def __init__(self, folder: str, dtype: torch.dtype = torch.float64, rounded: bool = False):
+        """``rounded``: what goes into a linear map and what comes out is rounded to bfloat16 (how far rounding alone moves a row)."""
         from safetensors.torch import load_file
         with open(os.path.join(folder, "config.json"), encoding="utf-8") as fh:
             self.cfg = json.load(fh)
-        self.dtype = dtype
+        self.dtype, self.rounded = dtype, rounded
         self.w: Dict[str, torch.Tensor] = {k: v.to(dtype) for k, v in load_file(os.path.join(folder, "model.safetensors")).items()}
         self.eps = float(self.cfg["norm"]["eps"])
 
     def lin(self, name: str, h: torch.Tensor, bias: bool = False) -> torch.Tensor:
-        y = h @ self.w[name].T
-        return y + self.w[name + ".b"] if bias else y
+        if self.rounded:
+            h = h.to(torch.bfloat16).to(self.dtype)
+        y = h @ self.w[name].T + (self.w[name + ".b"] if bias else 0.0)
+        return y.to(torch.bfloat16).to(self.dtype) if self.rounded else y
 
     def attention(self, p: str, m: dict, h: torch.Tensor, pos: torch.Tensor) -> torch.Tensor:
         T, H, G, d, e = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
@@ -180,7 +183,9 @@ class PlainVarolix:
         T, H, d, e, cap = h.shape[0], m["heads"], m["dim"], m["vdim"], float(m["gate_cap"])
         q, k = (self.lin(p + "q", h) * d ** -0.5).view(T, H, d), self.lin(p + "k", h).view(T, H, d)
         v = self.lin(p + "v", h).view(T, H, e)
-        i, f = log_input_gate(self.lin(p + "i", h, True), cap), log_forget_gate(self.lin(p + "f", h, True), cap)
+        # (the gates' logits are not rounded: they enter the recurrence)
+        zi, zf = (h @ self.w[p + n].T + self.w[p + n + ".b"] for n in ("i", "f"))
+        i, f = log_input_gate(zi, cap), log_forget_gate(zf, cap)
         o = torch.stack([matrix_memory(q[:, a], k[:, a], v[:, a], i[:, a], f[:, a])[0] for a in range(H)], dim=1)
         o = unit_rms(o, self.eps).reshape(T, H * e) * self.w[p + "norm"] * torch.sigmoid(self.lin(p + "g", h))
         return self.lin(p + "o", o)
