@@ -406,6 +406,15 @@ int bc4g_attention_maps(const float* q, long q_row, const void* k_cache, const v
                         int vdim, int page_tokens, int window, int keep_first, float scale, int waves, const float* sink,
                         const float* far1, const float* far2, int block, float cap, const float* point, void* stream);
 
+// The same with one map, on the matrix cores (attention_heads_mfma.hip), for a bfloat16 cache and dim, vdim multiples of 8 up to
+// 256: every float32 query element and weight enters as three bfloat16 numbers whose sum it is, so that scores, weights and
+// sums stay 32-bit.  The step's rows grouped by request (seq_start [S + 1], seq_ctx [S]: tokens cached before the step);
+// most_rows: the most rows one request brings.  out's rows lie out_row elements apart.
+int bc4g_attention_heads_mfma(const float* q, long q_row, const void* k_cache, const void* v_cache, const int32_t* block_table,
+                              int table_stride, const int32_t* seq_start, const int32_t* seq_ctx, int n_seqs, int most_rows, void* out,
+                              int out_dtype, long out_row, int n_heads, int n_kv_heads, int dim, int vdim, int page_tokens, int window,
+                              float scale, const float* sink, float factor, void* stream);
+
 // Windowed softmax attention whose heads' weights are mixed before they meet the values (attention_talk.hip): q float32
 // [T, heads, dim]; keys [page, kv_head, token, dim], values [page, kv_head, token, vdim]; a row at p sees j <= p with
 // p - j < window (0: all).  score = q . k * scale - far1 ln(1 + far2 (p - j)); w_g = exp(score_g) / (sum_j exp(score_g)

@@ -66,6 +66,7 @@ _SIGNATURES = {
     "bc4g_heads_finish": [_P, _P, _F, _F, _P, _I, c_long, _I, _P, _I, _I, _I, _I, _P],
     "bc4g_decay_scan": [_P, _I, c_long, _F, _P, _I, c_long, _P, _I, c_long, _P, _P, _I, c_long, _P, _F, _P, _P, _P, _P, _P, _P, _P,
                         _I, _I, _I, _I, _I, _I, _P],
+    "bc4g_attention_heads_mfma": [_P, c_long, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, c_long, _I, _I, _I, _I, _I, _I, _F, _P, _F, _P],
     "bc4g_matrix_memory": [_P, _P, _P, _P, _P, _P, _I, c_long, _P, _P, _F, _F, _P, _F, _F, _P, _I, c_long, _P, _P, _P, _P, _P, _P, _P,
                            _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "bc4g_attention_maps": [_P, c_long, _P, _P, _I, _P, _I, _P, _P, _F, _I, _F, _F, _P, _I, c_long, _I, _P, _I,

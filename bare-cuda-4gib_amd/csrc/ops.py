@@ -1652,6 +1652,8 @@ DECAY_SCAN_CHUNK = 32       # rows of a request that one workgroup of the scan w
 
 ACT_NONE, ACT_SILU, ACT_SIGMOID = 0, 1, 2
 ATTENTION_MAPS_FULL = 4096   # (row, head) pairs from which on one wave walks a row's keys alone
+ATTENTION_HEADS_MFMA = True  # (off: the plain kernel also where the matrix-core kernel takes the call)
+ATTENTION_HEADS_ROWS = 64    # rows of one request x query heads a key/value head from which on the matrix-core kernel takes a step: a workgroup's
 
 
 def _part_of_rows(what: str, name: str, t: torch.Tensor, width: int) -> int:
@@ -1888,6 +1890,13 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch
     return out
 
 
+def attention_heads_mfma_takes(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor) -> bool:
+    """Whether the matrix-core kernel behind attention_maps serves these operands (one map, no option but window, sink and factor)."""
+    dim, vdim = k_cache.shape[3], v_cache.shape[3]
+    return (k_cache.dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0 and dim <= 256 and vdim <= 256
+            and all(t.data_ptr() % 16 == 0 for t in (q, k_cache, v_cache)))
+
+
 def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, ctx, out_dtype: torch.dtype,
                    n_heads: int, n_kv_heads: int, maps: int, dim: int, vdim: int, window: int, keep_first: int, scale: float, *,
                    lam: float = 0.0, normalize: bool = False, eps: float = 0.0, factor: float = 1.0,
@@ -1899,6 +1908,8 @@ def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     [T, n_heads, maps, dim]; keys [pages, n_kv_heads * maps, page_tokens, dim], values [pages, n_kv_heads, page_tokens, vdim].
     A row at position p sees key j <= p if p - j < window or j < keep_first (window 0: every key).  o = a1 - lam a2,
     with ``normalize`` divided by sqrt(mean(o^2) + eps) over the head, times ``factor`` and act(gate); [T, n_heads * vdim].
+    Steps that bring many rows of a request with one map, a bfloat16 cache and no option but window, sink and factor go to the
+    matrix-core kernel (attention_heads_mfma.hip: the same 32-bit arithmetic in another order).
     ``waves``: how many waves cut one row's keys among them (0: chosen here -- one where the rows fill the GPU, up to
     eight where few rows walk long contexts).  ``sink`` (float32 [n_heads]): exp(sink) joins every map's denominator, with
     no key and no value.  ``far`` = (r1, r2), float32 [n_heads] each: r1 ln(1 + r2 (p - j)) is taken off the scaled score.
@@ -1945,6 +1956,16 @@ def attention_maps(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
                 keys += cached + new
         return (2.0 * pairs * n_heads * maps * (dim + vdim),
                 keys * n_kv_heads * (maps * dim + vdim) * k_cache.element_size() + t * n_heads * (4 * maps * dim + vdim * out.element_size()))
+    most = max((int(ctx.seq_start[s + 1] - ctx.seq_start[s]) for s in range(ctx.n_seqs)), default=0)
+    if (ATTENTION_HEADS_MFMA and waves <= 0 and maps == 1 and not normalize and gate is None and not far and block == 0 and cap == 0
+            and point is None and (keep_first == 0 or window == 0) and attention_heads_mfma_takes(q, k_cache, v_cache)
+            and most > 1 and most * (n_heads // n_kv_heads) >= ATTENTION_HEADS_ROWS):
+        _i32("attention_maps", "seq_start", ctx.seq_start_dev, ctx.n_seqs + 1)
+        _i32("attention_maps", "seq_ctx", ctx.seq_ctx_dev, ctx.n_seqs)
+        library.call("bc4g_attention_heads_mfma", _ptr(q), n_heads * dim, _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.stride(0),
+                     _ptr(ctx.seq_start_dev), _ptr(ctx.seq_ctx_dev), ctx.n_seqs, most, _ptr(out), _code(out, "attention_maps"), out_row,
+                     n_heads, n_kv_heads, dim, vdim, page_tokens, int(window), float(scale), _ptr(sink), float(factor), _stream(), cost=cost)
+        return out
     if waves <= 0:
         reach = min(ctx.max_kv_len, block) if block > 0 else ctx.max_kv_len if window <= 0 else min(ctx.max_kv_len, window + keep_first)
         tiles = max(1, -(-reach // 64))

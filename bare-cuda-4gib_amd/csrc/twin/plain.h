@@ -48,6 +48,8 @@ inline double squared_relu(double z) { return z > 0.0 ? z * z : 0.0; }
 
 // silu(g) * u, silu(g) = g / (1 + exp(-g)) (reference: engine/kernels/swiglu.cu:22-23).
 inline double swiglu(double g, double u) { return g / (1.0 + std::exp(-g)) * u; }
+// The same with the gelu written with tanh.
+inline double geglu(double g, double u) { return 0.5 * g * (1.0 + std::tanh(std::sqrt(2.0 / 3.14159265358979323846) * (g + 0.044715 * g * g * g))) * u; }
 
 // One row's causal attention: scores q.k / sqrt(d) over keys lo .. pos, softmax, weighted sum of the values
 // (reference: engine/kernels/attention_qk.cu:25-68, softmax.cu:28-42, attention_av.cu:32-45).  keys/values:

@@ -117,12 +117,13 @@ bool swiglu() {
   const std::vector<float> gu = normals(rng, static_cast<size_t>(n) * 2 * inter, 2.0f);
   bool ok = true;
   for (int dtype = 0; dtype < 2; ++dtype)
-    for (int interleaved = 0; interleaved < 2; ++interleaved) {
+    for (int form = 0; form < 4; ++form) {
+      const int interleaved = form % 2, act = form / 2;
       const std::vector<double> in = dtype ? widen(as_bf16(gu)) : widen(gu);
       Dev<float> g32(gu), o32(static_cast<size_t>(n) * inter);
       Dev<bf16> g16(as_bf16(gu)), o16(static_cast<size_t>(n) * inter);
       RUN(bc4g_swiglu(dtype ? static_cast<const void*>(g16.p) : g32.p, dtype ? static_cast<void*>(o16.p) : o32.p, dtype, n,
-                      inter, interleaved, 0, kStream));
+                      inter, interleaved, act, kStream));
       std::vector<double> want;
       for (int t = 0; t < n; ++t)
         for (int i = 0; i < inter; ++i) {
@@ -130,9 +131,9 @@ bool swiglu() {
           // interleaved: blocks of 16 = eight gates, then the eight ups of the same outputs
           const size_t g = interleaved ? row + (i / 8) * 16 + i % 8 : row + i;
           const size_t u = interleaved ? g + 8 : row + inter + i;
-          want.push_back(plain::swiglu(in[g], in[u]));
+          want.push_back(act ? plain::geglu(in[g], in[u]) : plain::swiglu(in[g], in[u]));
         }
-      ok &= close(interleaved ? "interleaved" : "gates then ups", dtype ? widen(o16.get()) : widen(o32.get()), want,
+      ok &= close(act ? "gelu" : interleaved ? "interleaved" : "gates then ups", dtype ? widen(o16.get()) : widen(o32.get()), want,
                   dtype ? kBf16 : 1e-5, 1e-6);
     }
   return ok;
@@ -144,15 +145,15 @@ bool gemm_generic() {
   const int n = 33, k = 50;
   for (int m : {3, 20}) {            // the small tile (a decode step) and the large one
     const std::vector<float> a = normals(rng, static_cast<size_t>(m) * k), w = normals(rng, static_cast<size_t>(n) * k);
-    const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n);
+    const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n), bias = normals(rng, n);
     {   // float x float -> float, and added into a float output
-      Dev<float> da(a), dw(w), out(static_cast<size_t>(m) * n), acc(before);
+      Dev<float> da(a), dw(w), db(bias), out(static_cast<size_t>(m) * n), acc(before);
       RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, out.p, 0, 0, nullptr, m, n, k, kStream));
-      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, acc.p, 0, 1, nullptr, m, n, k, kStream));
+      RUN(bc4g_gemm_generic(da.p, 0, dw.p, 0, acc.p, 0, 1, db.p, m, n, k, kStream));
       const std::vector<double> want = plain::gemm(widen(a), widen(w), m, n, k);
       ok &= close("float product", widen(out.get()), want, 1e-5, 1e-5);
       std::vector<double> sum = want;
-      for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i];
+      for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i] + bias[i % n];
       ok &= close("float product added", widen(acc.get()), sum, 1e-5, 1e-5);
     }
     {   // bfloat16 x bfloat16 -> float
@@ -173,29 +174,32 @@ bool gemm_skinny() {
   Dev<bf16> packed(pack_weight(w, n, k));
   for (int m : {1, 9, 33, 64}) {
     const std::vector<bf16> x = as_bf16(normals(rng, static_cast<size_t>(m) * k));
-    const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n);
+    const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n), bias = normals(rng, n);
     const std::vector<double> want = plain::gemm(widen(x), widen(w), m, n, k);
-    Dev<bf16> dx(x), o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2);
-    Dev<float> o32(static_cast<size_t>(m) * n), acc(before);
+    Dev<bf16> dx(x), o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2), gelu(static_cast<size_t>(m) * n / 2);
+    Dev<float> db(bias), o32(static_cast<size_t>(m) * n), acc(before);
     RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, nullptr, 0, m, n, k, kStream));
     RUN(bc4g_gemm_skinny(dx.p, packed.p, o32.p, nullptr, 1, m, n, k, kStream));
-    RUN(bc4g_gemm_skinny(dx.p, packed.p, acc.p, nullptr, 2, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, acc.p, db.p, 2, m, n, k, kStream));
     RUN(bc4g_gemm_skinny(dx.p, packed.p, act.p, nullptr, 3, m, n, k, kStream));
+    RUN(bc4g_gemm_skinny(dx.p, packed.p, gelu.p, nullptr, 7, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
     RUN(bc4g_gemm_skinny(dx.p, packed.p, o16.p, nullptr, 6, m, n, k, kStream));
     std::vector<double> squared = want;
     for (double& v : squared) v = plain::squared_relu(v);
     ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
     ok &= close("float out", widen(o32.get()), want, 1e-4, 1e-4);
-    std::vector<double> sum = want, gated;
-    for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i];
+    std::vector<double> sum = want, gated, gated_gelu;
+    for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i] + bias[i % n];
     ok &= close("added to a float stream", widen(acc.get()), sum, 1e-4, 1e-4);
     for (int r = 0; r < m; ++r)           // every 16 rows of w: eight gate rows, then the eight up rows of the same outputs
       for (int i = 0; i < n / 2; ++i) {
         const size_t g = static_cast<size_t>(r) * n + (i / 8) * 16 + i % 8;
         gated.push_back(plain::swiglu(want[g], want[g + 8]));
+        gated_gelu.push_back(plain::geglu(want[g], want[g + 8]));
       }
     ok &= close("SwiGLU", widen(act.get()), gated, kBf16, 1e-2);
+    ok &= close("gelu for the silu", widen(gelu.get()), gated_gelu, kBf16, 1e-2);
   }
   return ok;
 }
@@ -265,32 +269,35 @@ bool gemm_mfma() {
   bool ok = true;
   const int m = 150, n = 192, k = 128;
   const std::vector<bf16> a = as_bf16(normals(rng, static_cast<size_t>(m) * k)), w = as_bf16(normals(rng, static_cast<size_t>(n) * k, 0.5f));
-  const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n);
+  const std::vector<float> before = normals(rng, static_cast<size_t>(m) * n), bias = normals(rng, n);
   const std::vector<double> want = plain::gemm(widen(a), widen(w), m, n, k);
   Dev<bf16> da(a), rows(w), packed(pack_weight(w, n, k));
   for (int w_packed = 0; w_packed < 2; ++w_packed) {       // the weight by rows (tiles staged through registers) and packed (straight into LDS)
     const void* dw = w_packed ? packed.p : rows.p;
-    Dev<bf16> o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2);
-    Dev<float> o32(static_cast<size_t>(m) * n), acc(before);
+    Dev<bf16> o16(static_cast<size_t>(m) * n), act(static_cast<size_t>(m) * n / 2), gelu(static_cast<size_t>(m) * n / 2);
+    Dev<float> db(bias), o32(static_cast<size_t>(m) * n), acc(before);
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, nullptr, 0, m, n, k, kStream));
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o32.p, nullptr, 1, m, n, k, kStream));
-    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, acc.p, nullptr, 2, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, acc.p, db.p, 2, m, n, k, kStream));
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, act.p, nullptr, 3, m, n, k, kStream));
+    RUN(bc4g_gemm_mfma(da.p, dw, w_packed, gelu.p, nullptr, 7, m, n, k, kStream));
     ok &= close("bfloat16 out", widen(o16.get()), want, kBf16, 1e-2);
     RUN(bc4g_gemm_mfma(da.p, dw, w_packed, o16.p, nullptr, 6, m, n, k, kStream));
     std::vector<double> squared = want;
     for (double& v : squared) v = plain::squared_relu(v);
     ok &= close("squared relu", widen(o16.get()), squared, kBf16, 1e-2);
     ok &= close("float out", widen(o32.get()), want, 1e-4, 1e-4);
-    std::vector<double> sum = want, gated;
-    for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i];
+    std::vector<double> sum = want, gated, gated_gelu;
+    for (size_t i = 0; i < sum.size(); ++i) sum[i] += before[i] + bias[i % n];
     ok &= close("added to a float stream", widen(acc.get()), sum, 1e-4, 1e-4);
     for (int r = 0; r < m; ++r)
       for (int i = 0; i < n / 2; ++i) {
         const size_t g = static_cast<size_t>(r) * n + (i / 8) * 16 + i % 8;
         gated.push_back(plain::swiglu(want[g], want[g + 8]));
+        gated_gelu.push_back(plain::geglu(want[g], want[g + 8]));
       }
     ok &= close("SwiGLU", widen(act.get()), gated, kBf16, 1e-2);
+    ok &= close("gelu for the silu", widen(gelu.get()), gated_gelu, kBf16, 1e-2);
   }
   // k cut into parts over workgroups, and the kernel that adds the parts to the stream and norms it
   const int rows_few = 20, width = 128, depth = 256, parts = 2;

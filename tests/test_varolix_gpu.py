@@ -463,6 +463,72 @@ def test_attention_over_every_key_finds_one_among_hundreds(dtype, sizes, needle)
                 assert float(w[needle]) > 0.9
 
 
+def plain_heads(q, k, v, positions, window, sink, scale, factor):
+    """q [T, H, d], one request's k [n, G, d], v [n, G, e]; row t stands at positions[t] -> [T, H * e] (float64)."""
+    T, H = q.shape[:2]
+    hg = H // k.shape[1]
+    out = []
+    for t in range(T):
+        p = int(positions[t])
+        lo = max(0, p - window + 1) if window else 0
+        row = []
+        for a in range(H):
+            s = (k[lo:p + 1, a // hg].double() @ q[t, a].double()) * scale
+            top = max(float(s.max()), float(sink[a]) if sink is not None else -math.inf)
+            e = torch.exp(s - top)
+            total = e.sum() + (math.exp(float(sink[a]) - top) if sink is not None else 0.0)
+            row.append((e @ v[lo:p + 1, a // hg].double()) / total * factor)
+        out.append(torch.cat(row))
+    return torch.stack(out)
+
+
+# heads, key/value heads, key and value sizes: every form of the matrix-core kernel, sizes it fills and sizes it pads, groups of
+# heads that do not divide sixteen rows
+FORMS = [(4, 4, 8, 8), (6, 2, 32, 40), (8, 1, 24, 128), (3, 1, 64, 200), (4, 2, 40, 24), (5, 5, 64, 64), (12, 3, 56, 128), (2, 1, 48, 256),
+         (4, 2, 128, 16), (7, 1, 104, 64), (8, 2, 128, 128), (2, 2, 72, 136), (3, 3, 256, 32), (4, 1, 136, 48), (6, 2, 200, 104), (20, 1, 256, 256)]
+
+
+@pytest.mark.parametrize("sizes", FORMS)
+@pytest.mark.parametrize("window,page", [(0, 16), (0, 12), (1, 16), (33, 8), (64, 64), (100, 16)])
+def test_attention_of_prompt_portions_on_the_matrix_cores_is_32_bit(sizes, window, page):
+    """Three requests in one step -- a whole prompt, a portion far in whose windows have left pages behind (NaN, no page in
+    the table), two rows -- against float64 at float32's accuracy, though the cache is bfloat16: large scores, a sink that
+    takes some of the weight and heads without one; the plain kernel computes the same."""
+    from bare_cuda_4gib_amd.csrc import ops
+    H, G, d, e = sizes
+    torch.manual_seed(d + window)
+    lengths, cached, scale, factor, n_pages = [90, 77, 2], [0, 140, 50], 0.6, 1.7, 60
+    perm, tables, seqs, at = torch.randperm(n_pages), torch.full((3, 30), -1, dtype=torch.int32), [], 0
+    kc = torch.full((n_pages, G, page, d), float("nan"), dtype=torch.bfloat16)
+    vc = torch.full((n_pages, G, page, e), float("nan"), dtype=torch.bfloat16)
+    for s, (new, old) in enumerate(zip(lengths, cached)):
+        k, v = (torch.randn(new + old, G, d) * (6.0 / math.sqrt(d))).bfloat16(), torch.randn(new + old, G, e).bfloat16()
+        pages = perm[at:at + -(-(new + old) // page)]
+        at += len(pages)
+        gone = (max(0, old - window + 1) // page) if window else 0
+        for j in range(gone * page, new + old):
+            kc[pages[j // page], :, j % page], vc[pages[j // page], :, j % page] = k[j], v[j]
+        tables[s, :len(pages)] = pages.to(torch.int32)
+        tables[s, :gone] = -1
+        seqs.append((k, v))
+    q = torch.randn(sum(lengths), H, d)
+    sink = torch.randn(H) * 3.0 + 4.0
+    ctx = step_context(lengths, cached, [0, 1, 2])
+    operands = q.view(-1, H, 1, d).to(DEV), kc.to(DEV), vc.to(DEV), tables.to(DEV)
+    for sk in (None, sink):
+        how = dict(sink=sk.to(DEV) if sk is not None else None, factor=factor)
+        got = ops.attention_maps(*operands, ctx, torch.float32, H, G, 1, d, e, window, 0, scale, **how).cpu().double()
+        other = ops.attention_maps(*operands, ctx, torch.float32, H, G, 1, d, e, window, 0, scale, waves=1, **how).cpu().double()
+        assert window == 1 or not torch.equal(got, other)       # (two kernels; with one key there is one sum)
+        row = 0
+        for s, (new, old) in enumerate(zip(lengths, cached)):
+            some = sorted({0, 1, new - 1, new // 2, min(new - 1, 63), min(new - 1, 31)})
+            want = plain_heads(q[[row + t for t in some]], *seqs[s], [old + t for t in some], window, sk, scale, factor)
+            for a, b in ((got, 1e-5), (other, 1e-5)):
+                assert torch.allclose(a[[row + t for t in some]], want, atol=b, rtol=b), (s, sk is not None)
+            row += new
+
+
 @pytest.mark.parametrize("dtype", BOTH)
 @pytest.mark.parametrize("sizes", [(3, 8, 6, 20, 14), (2, 4, 2, 9, 300), (4, 16, 32, 64, 24)])
 def test_latents_turned_in_halves_and_the_queries_own_latent(dtype, sizes):
