@@ -297,7 +297,7 @@ def fresh_state(slots, H, d, e):
 
 
 # one number of everything; every bucket of the scan's registers; values of one to four waves; sizes of 16-byte pieces and not
-MEMORIES = [(1, 1, 2), (3, 5, 3), (2, 16, 16), (3, 17, 64), (2, 48, 48), (2, 64, 128), (1, 100, 130), (2, 128, 128), (1, 200, 256), (2, 256, 65)]
+MEMORIES = [(1, 1, 2), (3, 5, 3), (2, 16, 16), (3, 17, 64), (3, 40, 36), (2, 64, 128), (1, 100, 130), (2, 128, 128), (1, 200, 256), (2, 256, 65)]
 
 
 @pytest.mark.parametrize("dtype", BOTH)
@@ -343,7 +343,7 @@ def test_the_memory_keeps_one_token_among_hundreds(dtype, sizes, marked):
     decoded, read that token's value; rows ahead of it read nothing of it.  A closed forget gate later takes it away."""
     H, d, e = sizes
     torch.manual_seed(marked)
-    n, cap = 300, 12.0
+    n, cap = 300, 11.0
     x = torch.randn(n, H * (2 * d + 2 * e) + 2 * H)
     x[:, -2 * H:-H], x[:, -H:] = -40.0, 60.0                      # i near -cap, f near 0
     x[marked, -2 * H:-H] = 40.0                                   # i near cap
@@ -427,7 +427,7 @@ def paged_heads(rows, pages, P, dtype, n_pages):
 
 
 @pytest.mark.parametrize("dtype", BOTH)
-@pytest.mark.parametrize("sizes", [(4, 2, 12, 10), (8, 2, 64, 128), (6, 6, 32, 64), (3, 1, 130, 70), (16, 4, 128, 128), (2, 1, 96, 48), (8, 1, 16, 16)])
+@pytest.mark.parametrize("sizes", [(4, 2, 12, 10), (8, 4, 64, 128), (6, 6, 32, 64), (3, 1, 130, 70), (16, 4, 128, 128), (2, 1, 96, 48), (8, 1, 16, 16)])
 @pytest.mark.parametrize("needle", [0, 15, 16, 31, 32, 63, 64, 120, 299])
 def test_attention_over_every_key_finds_one_among_hundreds(dtype, sizes, needle):
     """No window: one key made to stand out, at the sequence's first place, at page and tile borders and the row's own, for

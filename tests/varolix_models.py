@@ -76,7 +76,7 @@ CONFIGS: Dict[str, dict] = {
     # widths at which the products take their matrix-core forms: multiples of 64, a prompt of a few hundred rows
     "F": dict(architecture="Varolix", vocab=320, width=192, norm=dict(eps=1e-5), loop=dict(start=1, stop=2, times=2), layers=[
         attention(6, 2, 32, 64, rot=16, scaling=(16.0, 128, 10.0, 1.0), ff=448),
-        parallel((6, 2, 32, 64), (4, 64, 64), 0.6, 0.8, temp=(0.3, 50), cap=12.0, ff=256),
+        parallel((6, 2, 32, 64), (4, 64, 64), 0.6, 0.8, temp=(0.25, 50), cap=11.0, ff=256),
         latent(6, 32, 32, 32, 64, 128, ff=192)]),
 }
 SEEDS = {"A": 11, "B": 22, "C": 33, "D": 44, "E": 55, "F": 66}
